@@ -15,7 +15,8 @@
 //   slope_exp E    s_j -= 2^(-E (h + 1) / H) * (p - j): a bias that grows with the distance, steeper for low heads;
 //   v_dim          the value size where it differs from the key size;
 //   values in the key pages (v_cache null): a layer whose values are its keys stores them once;
-//   out_scale      o is multiplied by it on store.
+//   out_scale      o is multiplied by it on store;
+//   sigmoid_bias   one float a query head: no softmax, P_j = sigmoid(s_j + bias_h), not normalised over the keys.
 //
 // K and V are read from the cache pages through the request's block table
 // (K page [Hkv][ceil(D / 8)][page][8], V page [Hkv][D][page]); the step's own tokens were
@@ -39,7 +40,7 @@ __global__ void __launch_bounds__(WAVES * 64) attn_paged_ref_kernel(
     const S* __restrict__ v_cache, const int32_t* __restrict__ block_table, int64_t max_blocks,
     const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ seq_lens, int num_reqs, float scale,
     int window, int H, int Hkv, int D, int page, int keep_first, const float* __restrict__ sinks, float slope_exp,
-    int Dv, float out_scale) {
+    int Dv, float out_scale, const float* __restrict__ sigmoid_bias) {
   __shared__ float qs[WAVES][MAX_D];
   __shared__ float ps[WAVES][64];
   const int t = blockIdx.x;
@@ -61,6 +62,7 @@ __global__ void __launch_bounds__(WAVES * 64) attn_paged_ref_kernel(
   const int hk = live ? h / (H / Hkv) : 0;
   const int Dp = (D + 7) & ~7;  // a head's keys fill whole 8-entry pieces of a page (the last one padded)
   const float slope = slope_exp != 0.f ? exp2f(-slope_exp * (float)(h + 1) / (float)H) : 0.f;
+  const float sb = sigmoid_bias && live ? sigmoid_bias[h] : 0.f;
   // two runs of keys: the kept first ones that the window has passed, then the window itself
   const int kept = keep_first < first_key ? keep_first : first_key;
 
@@ -88,11 +90,16 @@ __global__ void __launch_bounds__(WAVES * 64) attn_paged_ref_kernel(
       for (int d = 0; d < D; ++d) acc += qs[wave][d] * to_f32(kr[k_page_offset(off, d, page)]);
       s = acc * scale - slope * (float)(p - j);
     }
-    const float m_new = fmaxf(m, wave_max(s));
-    const float pj = (live && j <= last) ? expf(s - m_new) : 0.f;
-    const float alpha = expf(m - m_new);  // m = -inf on the first tile: alpha = 0
-    l = l * alpha + wave_sum(pj);
-    m = m_new;
+    float pj, alpha = 1.f;
+    if (sigmoid_bias) {
+      pj = (live && j <= last) ? 1.f / (1.f + expf(-(s + sb))) : 0.f;
+    } else {
+      const float m_new = fmaxf(m, wave_max(s));
+      pj = (live && j <= last) ? expf(s - m_new) : 0.f;
+      alpha = expf(m - m_new);  // m = -inf on the first tile: alpha = 0
+      l = l * alpha + wave_sum(pj);
+      m = m_new;
+    }
     __syncthreads();  // the previous tile's ps[] has been consumed
     ps[wave][lane] = pj;
     __syncthreads();
@@ -125,7 +132,7 @@ __global__ void __launch_bounds__(WAVES * 64) attn_paged_ref_kernel(
   }
   if (live) {
     S* orow = out + (int64_t)t * ld_out + (int64_t)h * Dv;
-    const float inv = l > 0.f ? out_scale / l : 0.f;
+    const float inv = sigmoid_bias ? out_scale : l > 0.f ? out_scale / l : 0.f;
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
       const int d = lane + 64 * c;
@@ -291,7 +298,7 @@ extern "C" int dinfer_attn_paged_ref(int dtype, const void* q, int64_t ld_q, voi
   DINFER_DISPATCH_DTYPE(dtype, {
     attn_paged_ref_kernel<S><<<grid, WAVES * 64, 0, stream>>>(
         (const S*)q, ld_q, (S*)out, ld_out, (const S*)k_cache, (const S*)v_cache, block_table, max_blocks, cu_seqlens,
-        seq_lens, num_reqs, scale, window, heads, kv_heads, head_dim, page_size, 0, nullptr, 0.f, head_dim, 1.f);
+        seq_lens, num_reqs, scale, window, heads, kv_heads, head_dim, page_size, 0, nullptr, 0.f, head_dim, 1.f, nullptr);
   });
   return launch_status();
 }
@@ -303,18 +310,19 @@ extern "C" int dinfer_attn_paged_ext(int dtype, const void* q, int64_t ld_q, voi
                                      int64_t max_blocks, const int32_t* cu_seqlens, const int32_t* seq_lens,
                                      int num_reqs, int64_t tokens, float scale, int window, int keep_first,
                                      const float* sinks, float slope_exp, int heads, int kv_heads, int head_dim,
-                                     int v_dim, int page_size, float out_scale, hipStream_t stream) {
+                                     int v_dim, int page_size, float out_scale, const float* sigmoid_bias,
+                                     hipStream_t stream) {
   if (tokens <= 0 || num_reqs <= 0) return OK;
   if (heads <= 0 || kv_heads <= 0 || heads % kv_heads != 0 || head_dim <= 0 || v_dim <= 0 || page_size <= 0 ||
       max_blocks <= 0 || window < 0 || keep_first < 0 || tokens > 0x7fffffff || (!v_cache && v_dim != head_dim))
     return ERR_BAD_SHAPE;
-  if (head_dim > MAX_D || v_dim > MAX_D) return ERR_UNSUPPORTED;
+  if (head_dim > MAX_D || v_dim > MAX_D || (sigmoid_bias && sinks)) return ERR_UNSUPPORTED;
   const dim3 grid((unsigned)tokens, (unsigned)((heads + WAVES - 1) / WAVES));
   DINFER_DISPATCH_DTYPE(dtype, {
     attn_paged_ref_kernel<S><<<grid, WAVES * 64, 0, stream>>>(
         (const S*)q, ld_q, (S*)out, ld_out, (const S*)k_cache, (const S*)v_cache, block_table, max_blocks, cu_seqlens,
         seq_lens, num_reqs, scale, window, heads, kv_heads, head_dim, page_size, window > 0 ? keep_first : 0, sinks,
-        slope_exp, v_dim, out_scale);
+        slope_exp, v_dim, out_scale, sigmoid_bias);
   });
   return launch_status();
 }

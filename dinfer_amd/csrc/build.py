@@ -29,6 +29,7 @@ SOURCES = {
     "rope": "rope.hip",
     "attention_ref": "attention_ref.hip",
     "attention": "attention.hip",
+    "attention_ext": "attention_ext.hip",
     "gemm_ref": "gemm_ref.hip",
     "gemm": "gemm.hip",
     "gemm_mid": "gemm_mid.hip",
@@ -37,14 +38,16 @@ SOURCES = {
     "grouped": "grouped.hip",
     "delta": "delta.hip",
     "decay": "decay.hip",
+    "linear_attention": "linear_attention.hip",
+    "scan": "scan.hip",
     "streams": "streams.hip",
     "sampling": "sampling.hip",
     "ceilings": "ceilings.hip",
     "host": "host/api.cpp",
 }
 HEADERS = ["common.cuh"]
-# headers of single libraries (their C interface), hashed with them
-OWN_HEADERS = {"gemm_mid": ["gemm_mid.h"]}
+# headers of single libraries (their C interface, or device code two of them share), hashed with them
+OWN_HEADERS = {"gemm_mid": ["gemm_mid.h"], "attention": ["attention_tile.cuh"], "attention_ext": ["attention_tile.cuh"]}
 # libraries without device code, and the headers each is made of
 HOST_ONLY = {"host": ["host/dinfer_host.h", "host/errors.hpp", "host/block_pool.hpp", "host/cache_manager.hpp",
                       "host/step_batch.hpp", "host/scheduler.hpp"]}

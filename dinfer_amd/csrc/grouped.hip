@@ -10,6 +10,8 @@
 //            or, with c_to_perm, to the entry. The work list `tiles` names (expert, first sorted place) of every
 //            row tile; entries beyond the step's tiles hold -1 and their workgroups leave at once.
 // GATED: W_g = [gate rows; up rows] stacked, gate_n rows each, and C = silu(A Wgate^T) * (A Wup^T).
+// row_scale (experts): the row of A belonging to entry e is multiplied by row_scale[e]; the product being linear in it, the
+// float sums are, before the activation.
 //
 // Float operands run on the vector ALUs, every output element summed over k in ascending order by one thread (the
 // true 32-bit path; a row's result does not depend on which tile or group size it met). bf16 operands run on the
@@ -20,7 +22,8 @@
 //                token the `top` largest (lowest index first among equals), the softmax over the chosen and the shared
 //                expert's sigmoid gate
 //   moe_scatter  counts, offsets, the sorted list and the work list, one workgroup (LDS counters)
-//   moe_combine  out[t] = sum_c share[t, c] * y[t * top + c] + shared_gate[t] * shared[t]   (no gate: + shared[t])
+//   moe_combine  out[t] = sum_c share[t, c] * y[t * top + c] + shared_gate[t] * shared[t]   (no gate: + shared[t]; no
+//                shares: every row of y counts as it is)
 #include "common.cuh"
 
 using namespace dinfer;
@@ -40,7 +43,8 @@ struct Groups {
   const void* gate; int64_t ld_gate;   // heads: optional
   int gate_n;               // GATED: rows of each half of W_g
   int tm;                   // rows of a tile: 64 on the vector ALUs, 16 or 128 on the matrix cores
-  int act;                  // not GATED: 0 nothing, 1 silu, 2 gelu (error function) on every result
+  int act;                  // not GATED: 0 nothing, 1 silu, 2 gelu (error function), 3 the square of relu on every result
+  const float* row_scale;   // experts: a factor an entry on its row of A, or null
 };
 
 __device__ __forceinline__ float silu(float x) { return x / (1.f + expf(-x)); }
@@ -48,6 +52,7 @@ __device__ __forceinline__ float sigmoid(float x) { return 1.f / (1.f + expf(-x)
 __device__ __forceinline__ float plain_act(float x, int act) {
   if (act == 1) return silu(x);
   if (act == 2) return 0.5f * x * (1.f + erff(x * 0.7071067811865476f));
+  if (act == 3) return x > 0.f ? x * x : 0.f;
   return x;
 }
 
@@ -77,6 +82,7 @@ struct Tile {
   }
   __device__ __forceinline__ int64_t a_row(int r) const { return perm && a_div > 0 ? perm[base + r] / a_div : base + r; }
   __device__ __forceinline__ int64_t c_row(int r) const { return perm && c_to_perm ? perm[base + r] : base + r; }
+  __device__ __forceinline__ float scale_of(const Groups& p, int r) const { return p.row_scale ? p.row_scale[perm[base + r]] : 1.f; }
 };
 
 template <class S, class O, bool GATED>
@@ -142,11 +148,12 @@ __global__ void __launch_bounds__(256) grouped_valu_kernel(Groups p) {
     const int64_t cr = tl.c_row(r);
     float g = 1.f;
     if (p.gate) g = sigmoid(to_f32(((const S*)p.gate)[cr * p.ld_gate + tl.z]));
+    const float rs = tl.scale_of(p, r);
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int gn = n0 + tx * 4 + j;
       if (gn < p.N) {
-        float v = GATED ? silu(acc[i][j]) * acu[i][j] : plain_act(acc[i][j], p.act);
+        float v = GATED ? silu(acc[i][j] * rs) * (acu[i][j] * rs) : plain_act(acc[i][j] * rs, p.act);
         C[cr * p.ldc + gn] = from_f32<O>(v * g);
       }
     }
@@ -254,11 +261,12 @@ __global__ void __launch_bounds__(256) grouped_mfma_big_kernel(Groups p) {
       const int64_t cr = tl.c_row(row);
       float g = 1.f;
       if (p.gate) g = sigmoid((float)((const bf16*)p.gate)[cr * p.ld_gate + tl.z]);
+      const float rs = tl.scale_of(p, row);
 #pragma unroll
       for (int j = 0; j < (GATED ? 2 : 4); ++j) {
         const int gn = GATED ? n0 + wn * 32 + j * 16 + lr : n0 + wn * 64 + j * 16 + lr;
         if (gn < p.N) {
-          const float v = GATED ? silu(acc[i][j][r]) * acc[i][j + 2][r] : plain_act(acc[i][j][r], p.act);
+          const float v = GATED ? silu(acc[i][j][r] * rs) * (acc[i][j + 2][r] * rs) : plain_act(acc[i][j][r] * rs, p.act);
           C[cr * p.ldc + gn] = from_f32<O>(v * g);
         }
       }
@@ -323,7 +331,8 @@ __global__ void __launch_bounds__(256) grouped_mfma_small_kernel(Groups p) {
   float g = 1.f;
   if (p.gate) g = sigmoid((float)((const bf16*)p.gate)[cr * p.ld_gate + tl.z]);
   O* C = (O*)p.C + (experts ? 0 : (int64_t)tl.z * p.c_zs);
-  C[cr * p.ldc + n0 + col] = from_f32<O>((GATED ? silu(v) * u : plain_act(v, p.act)) * g);
+  const float rs = tl.scale_of(p, row);
+  C[cr * p.ldc + n0 + col] = from_f32<O>((GATED ? silu(v * rs) * (u * rs) : plain_act(v * rs, p.act)) * g);
 }
 
 // ---- routing ---------------------------------------------------------------------------------------------------
@@ -397,6 +406,8 @@ __global__ void __launch_bounds__(256) moe_logits_bf16x8_kernel(const bf16* __re
 // over the chosen, and the sigmoid of the shared expert's gate logit (z[t, E]) where there is one.
 // all_scores: the scores are the softmax over all E logits; the choice goes by score + correction[e] (correction may
 // be null) and a chosen expert's weight is its score as it is (the weights of a token need not sum to one).
+// all_scores 2: the scores are the sigmoids of the logits one by one, chosen and weighing as they are (the sigmoid keeps
+// the logits' order, so the choice goes by the logits, which tie no sooner than they do).
 __global__ void __launch_bounds__(256) moe_topk_kernel(const float* __restrict__ z, int ldz, int tokens, int E, int top,
                                                        int has_shared, int32_t* __restrict__ idx,
                                                        float* __restrict__ share, float* __restrict__ shared_gate,
@@ -409,7 +420,7 @@ __global__ void __launch_bounds__(256) moe_topk_kernel(const float* __restrict__
   float* zw = zs[wave];
   for (int e = lane; e < E; e += 64) zw[e] = z[t * ldz + e];
   if (has_shared && lane == 0) shared_gate[t] = sigmoid(z[t * ldz + E]);
-  if (all_scores) {
+  if (all_scores == 1) {
     float* sw = sc[wave];
     float mx = -INFINITY;
     for (int e = lane; e < E; e += 64) mx = fmaxf(mx, zw[e]);   // (a lane reads back what it wrote itself)
@@ -475,7 +486,7 @@ __global__ void __launch_bounds__(256) moe_topk_kernel(const float* __restrict__
   }
   if (lane < top) {
     idx[t * top + lane] = chosen_e;
-    share[t * top + lane] = expf(chosen - zmax) / sum;
+    share[t * top + lane] = all_scores == 2 ? sigmoid(chosen) : expf(chosen - zmax) / sum;
   }
 }
 
@@ -530,7 +541,7 @@ __global__ void __launch_bounds__(256) moe_combine_kernel(const S* __restrict__ 
     for (int c = 0; c < top; ++c) {
       // an expert without weights hands the token's input on
       const bool same = idx && idx[t * top + c] >= real;
-      acc = fmaf(share[t * top + c], to_f32(same ? x[t * ld_x + i] : y[(t * top + c) * ld_y + i]), acc);
+      acc = fmaf(share ? share[t * top + c] : 1.f, to_f32(same ? x[t * ld_x + i] : y[(t * top + c) * ld_y + i]), acc);
     }
     if (shared) acc = fmaf(sg, to_f32(shared[t * ld_s + i]), acc);
     out[t * ld_o + i] = from_f32<S>(acc);
@@ -560,7 +571,7 @@ __global__ void __launch_bounds__(256) moe_combine_bf16x8_kernel(const bf16* __r
     for (int c = 0; c < top; ++c) {
       const bool same = idx && idx[t * top + c] >= real;   // an expert without weights hands the token's input on
       const bf16x8 v = *(const bf16x8*)(same ? x + t * ld_x + i : y + (t * top + c) * ld_y + i);
-      const float w = share[t * top + c];
+      const float w = share ? share[t * top + c] : 1.f;
 #pragma unroll
       for (int j = 0; j < 8; ++j) acc[j] = fmaf(w, (float)v[j], acc[j]);
     }
@@ -613,12 +624,12 @@ extern "C" int dinfer_heads_nt(int dtype, const void* A, int64_t lda, int64_t a_
 }
 
 // The products of the experts (see the head of the file). W [experts][rows][ldw] with w_zs elements an expert;
-// gated 1: rows = 2 N (gate rows, then up rows); 0: plain; 2, 3: plain with silu or gelu (error function) on every
-// result. max_tiles: the length of `tiles`.
+// gated 1: rows = 2 N (gate rows, then up rows); 0: plain; 2, 3, 4: plain with silu, gelu (error function) or the square of
+// relu on every result. max_tiles: the length of `tiles`. row_scale (may be null): float, a factor an entry on its row of A.
 extern "C" int dinfer_experts_nt(int dtype, int gated, const void* A, int64_t lda, const void* W, int64_t ldw,
                                  int64_t w_zs, void* C, int64_t ldc, int64_t N, int64_t K, const int32_t* tiles,
                                  int64_t max_tiles, int tile_rows, const int32_t* offsets, const int32_t* perm, int a_div,
-                                 int c_to_perm, hipStream_t stream) {
+                                 int c_to_perm, const float* row_scale, hipStream_t stream) {
   if (N <= 0 || max_tiles <= 0) return OK;
   if (K <= 0 || ldw < K || lda < K || ldc < N || N > 0x7fffffff || K > 0x7fffffff || max_tiles > 65535 || !tiles ||
       !offsets || !perm || tile_rows <= 0)
@@ -627,7 +638,8 @@ extern "C" int dinfer_experts_nt(int dtype, int gated, const void* A, int64_t ld
   p.A = A; p.lda = lda; p.W = W; p.ldw = ldw; p.w_zs = w_zs; p.C = C; p.ldc = ldc;
   p.N = (int)N; p.K = (int)K; p.tiles = tiles; p.offsets = offsets; p.perm = perm; p.a_div = a_div;
   p.c_to_perm = c_to_perm; p.gate_n = (int)N; p.tm = tile_rows;
-  if (gated < 0 || gated > 3) return ERR_UNSUPPORTED;
+  p.row_scale = row_scale;
+  if (gated < 0 || gated > 4) return ERR_UNSUPPORTED;
   p.act = gated >= 2 ? gated - 1 : 0;
   if (!mfma_fits(dtype, p) && tile_rows > BM) return ERR_UNSUPPORTED;
   return gated == 1 ? launch_groups<true>(dtype, p, (unsigned)max_tiles, 1, stream)
@@ -647,10 +659,11 @@ extern "C" int dinfer_moe_route(int dtype, const void* x, int64_t ld_x, int64_t 
                                 const float* shared_gate_w, int experts, int top, int width, float* z, int32_t* idx,
                                 float* share, float* shared_gate, int all_scores, const float* correction,
                                 hipStream_t stream) {
-  // all_scores: softmax over all experts, chosen by score + correction (float [experts] or null), weights the scores
+  // all_scores 1: softmax over all experts, chosen by score + correction (float [experts] or null), weights the scores;
+  // 2: the scores are sigmoids of the logits (no correction)
   if (tokens <= 0) return OK;
   if (experts <= 0 || top <= 0 || top > experts || width <= 0 || tokens > 0x7fffffff || !z) return ERR_BAD_SHAPE;
-  if (experts > MAX_EXPERTS || top > 64) return ERR_UNSUPPORTED;
+  if (experts > MAX_EXPERTS || top > 64 || (correction && all_scores != 1)) return ERR_UNSUPPORTED;
   const int rows = experts + (shared_gate_w ? 1 : 0), ldz = experts + 1;
   const int rt = tokens <= 128 ? 1 : 8;
   const dim3 grid((unsigned)((tokens + rt - 1) / rt), (unsigned)((rows + 3) / 4));
@@ -699,7 +712,7 @@ extern "C" int dinfer_moe_combine(int dtype, const void* y, int64_t ld_y, const 
                                   int width, const int32_t* idx, int real_experts, const void* x, int64_t ld_x,
                                   hipStream_t stream) {
   // idx (may be null) [tokens, top] with real_experts: a choice from real_experts on adds its share of x[t], the
-  // token's input, instead of a row of y.
+  // token's input, instead of a row of y. share null: every choice counts as it is.
   if (tokens <= 0) return OK;
   if (top <= 0 || width <= 0 || tokens > 0x7fffffff || (idx && (!x || ld_x < width))) return ERR_BAD_SHAPE;
   const bool vec = dtype == DT_BF16 && width % 8 == 0 && ld_y % 8 == 0 && ld_o % 8 == 0 && (!shared || ld_s % 8 == 0) &&

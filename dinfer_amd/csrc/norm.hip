@@ -491,3 +491,346 @@ extern "C" int dinfer_rmsnorm_stream(const void* branch, int branch_dtype, int64
       out_dtype, eps, off, width);
   return launch_status();
 }
+
+// ---- norms in groups, and branches that are normed before they are summed -----------------------------------------
+// group_rmsnorm: a row of `width` columns in `groups` equal consecutive parts, each divided by its own root mean square:
+//   stream[s] = round(stream[s] + x[s])                                                   (with a stream)
+//   out[r, c] = v[c] / sqrt(mean over c's part of v^2 + eps) * w[c],   v = stream[s] (or x[s])
+// joined_norms: M branches side by side in a row, each normed over its own `width` columns and then summed:
+//   y[c] = scale * sum_m (b_m[c] + bias_m[c]) / sqrt(mean (b_m + bias_m)^2 + eps_m) * w_m[c]
+//   out[r] = y,   or, with a stream:   stream[r] += y;   out[r] = group norm of stream[r]
+// Both keep the sums in float and round every stored value once.
+namespace {
+
+constexpr int MAX_GROUPS = 1024;
+constexpr int MAX_BRANCHES = 4;
+
+// inv[g] = 1 / sqrt(mean of part g of row[] + eps): a wave takes every fourth part. row and inv lie in LDS; the caller
+// has written row and not yet met a barrier.
+__device__ __forceinline__ void group_inverses(const float* row, float* inv, int width, int groups, float eps) {
+  const int part = width / groups, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  __syncthreads();
+  for (int g = wave; g < groups; g += (int)(blockDim.x >> 6)) {
+    float ss = 0.f;
+    for (int i = lane; i < part; i += 64) ss = add_square(ss, row[g * part + i]);
+    ss = wave_sum(ss);
+    if (lane == 0) inv[g] = 1.f / sqrtf(ss / (float)part + eps);
+  }
+  __syncthreads();
+}
+
+__global__ void __launch_bounds__(256) group_rmsnorm_kernel(const void* __restrict__ x, int x_dt, int64_t ld_x,
+                                                            void* __restrict__ stream, int s_dt, int64_t ld_s,
+                                                            const int32_t* __restrict__ rows, const float* __restrict__ w,
+                                                            void* __restrict__ out, int o_dt, float eps, int width,
+                                                            int groups) {
+  extern __shared__ float row[];
+  float* inv = row + width;
+  const int64_t r = blockIdx.x;
+  const int64_t s = rows ? (int64_t)rows[r] : r;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) {
+    float v = ld_any(x, s * ld_x + i, x_dt);
+    if (stream) {
+      v = round_any(v + ld_any(stream, s * ld_s + i, s_dt), s_dt);
+      st_any(stream, s * ld_s + i, s_dt, v);
+    }
+    row[i] = v;
+  }
+  group_inverses(row, inv, width, groups, eps);
+  const int part = width / groups;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) st_any(out, r * width + i, o_dt, row[i] * inv[i / part] * w[i]);
+}
+
+// 8 consecutive values of a row of either type, as floats
+__device__ __forceinline__ void load8(const bf16* p, float (&v)[8]) {
+  const bf16x8 t = *(const bf16x8*)p;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v[j] = (float)t[j];
+}
+__device__ __forceinline__ void load8(const float* p, float (&v)[8]) {
+  const f32x4 a = *(const f32x4*)p, b = *(const f32x4*)(p + 4);
+#pragma unroll
+  for (int j = 0; j < 4; ++j) { v[j] = a[j]; v[4 + j] = b[j]; }
+}
+__device__ __forceinline__ void store8(bf16* p, const float (&v)[8]) {
+  bf16x8 t;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) t[j] = (bf16)v[j];
+  *(bf16x8*)p = t;
+}
+__device__ __forceinline__ void store8(float* p, const float (&v)[8]) {
+  f32x4 a, b;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) { a[j] = v[j]; b[j] = v[4 + j]; }
+  *(f32x4*)p = a;
+  *(f32x4*)(p + 4) = b;
+}
+
+// The end both register kernels share: the row's pieces v (a thread's it-th piece is number it * 256 + thread), parts of
+// whole pieces. sums: [256 * ITERS] in LDS.
+template <class SO, int ITERS>
+__device__ __forceinline__ void group_norm_pieces(const float (&v)[ITERS][8], const float* __restrict__ w, SO* __restrict__ out,
+                                                  int n8, int groups, float eps, float* sums, float* inv) {
+  float g[ITERS][8];
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int i = it * 256 + threadIdx.x;
+    if (i < n8) {
+      load8(w + (int64_t)i * 8, g[it]);
+      float ss = 0.f;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss = add_square(ss, v[it][j]);
+      sums[i] = ss;
+    }
+  }
+  const int part = n8 / groups, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  __syncthreads();
+  for (int q = wave; q < groups; q += 4) {
+    float ss = 0.f;
+    for (int i = lane; i < part; i += 64) ss += sums[q * part + i];
+    ss = wave_sum(ss);
+    if (lane == 0) inv[q] = 1.f / sqrtf(ss / (float)(part * 8) + eps);
+  }
+  __syncthreads();
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int i = it * 256 + threadIdx.x;
+    if (i < n8) {
+      const float f = inv[i / part];
+      float y[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) y[j] = v[it][j] * f * g[it][j];
+      store8(out + (int64_t)i * 8, y);
+    }
+  }
+}
+
+// The combinations the engine meets: a row in registers from the first read to the last store, 16 or 32 bytes a move.
+template <class SX, class SO, int ITERS>
+__global__ void __launch_bounds__(256) group_rmsnorm_regs_kernel(const SX* __restrict__ x, int64_t ld_x,
+                                                                 float* __restrict__ stream, int64_t ld_s,
+                                                                 const int32_t* __restrict__ rows,
+                                                                 const float* __restrict__ w, SO* __restrict__ out,
+                                                                 float eps, int width, int groups) {
+  __shared__ float sums[256 * ITERS];
+  __shared__ float inv[MAX_GROUPS];
+  const int64_t r = blockIdx.x;
+  const int64_t s = rows ? (int64_t)rows[r] : r;
+  const int n8 = width / 8;
+  float v[ITERS][8];
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int i = it * 256 + threadIdx.x;
+    if (i < n8) {
+      load8(x + s * ld_x + (int64_t)i * 8, v[it]);
+      if (stream) {
+        float t[8];
+        load8(stream + s * ld_s + (int64_t)i * 8, t);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[it][j] += t[j];
+        store8(stream + s * ld_s + (int64_t)i * 8, v[it]);
+      }
+    }
+  }
+  group_norm_pieces<SO, ITERS>(v, w, out + r * width, n8, groups, eps, sums, inv);
+}
+
+struct Branches {
+  const float* w;      // [M][width]
+  const float* bias;   // [M][width] or null
+  float eps[MAX_BRANCHES];
+  int m;
+  int64_t stride;      // columns from one branch to the next
+  float scale;
+};
+
+template <class S>
+__global__ void __launch_bounds__(256) joined_norms_kernel(const S* __restrict__ x, int64_t ld_x, Branches br,
+                                                           float* __restrict__ stream, int64_t ld_s,
+                                                           const float* __restrict__ w, S* __restrict__ out, float eps,
+                                                           int width, int groups) {
+  extern __shared__ float row[];      // [width] sums, [groups] inverses
+  __shared__ float red[16];
+  float* inv = row + width;
+  const int64_t r = blockIdx.x;
+  for (int m = 0; m < br.m; ++m) {
+    const S* b = x + r * ld_x + m * br.stride;
+    const float* bias = br.bias ? br.bias + (int64_t)m * width : nullptr;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < width; i += blockDim.x) ss = add_square(ss, to_f32(b[i]) + (bias ? bias[i] : 0.f));
+    const float f = 1.f / sqrtf(block_sum(ss, red) / (float)width + br.eps[m]);
+    for (int i = threadIdx.x; i < width; i += blockDim.x) {      // (each thread re-reads what it wrote itself)
+      const float y = (to_f32(b[i]) + (bias ? bias[i] : 0.f)) * f * br.w[(int64_t)m * width + i];
+      row[i] = m ? row[i] + y : y;
+    }
+  }
+  if (!stream) {
+    for (int i = threadIdx.x; i < width; i += blockDim.x) out[r * width + i] = from_f32<S>(row[i] * br.scale);
+    return;
+  }
+  for (int i = threadIdx.x; i < width; i += blockDim.x) {
+    const float v = __builtin_fmaf(row[i], br.scale, stream[r * ld_s + i]);
+    stream[r * ld_s + i] = v;
+    row[i] = v;
+  }
+  if (!out) return;
+  group_inverses(row, inv, width, groups, eps);
+  const int part = width / groups;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) out[r * width + i] = from_f32<S>(row[i] * inv[i / part] * w[i]);
+}
+
+template <class S, int ITERS>
+__global__ void __launch_bounds__(256) joined_norms_regs_kernel(const S* __restrict__ x, int64_t ld_x, Branches br,
+                                                                float* __restrict__ stream, int64_t ld_s,
+                                                                const float* __restrict__ w, S* __restrict__ out,
+                                                                float eps, int width, int groups) {
+  __shared__ float sums[256 * ITERS];
+  __shared__ float inv[MAX_GROUPS];
+  __shared__ float red[16];
+  const int64_t r = blockIdx.x;
+  const int n8 = width / 8;
+  float v[ITERS][8], t[ITERS][8];
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {      // asked for before the branches' sums are awaited
+    const int i = it * 256 + threadIdx.x;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) { v[it][j] = 0.f; t[it][j] = 0.f; }
+    if (stream && i < n8) load8(stream + r * ld_s + (int64_t)i * 8, t[it]);
+  }
+  for (int m = 0; m < br.m; ++m) {
+    float b[ITERS][8];
+    float ss = 0.f;
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+      const int i = it * 256 + threadIdx.x;
+      if (i < n8) {
+        load8(x + r * ld_x + m * br.stride + (int64_t)i * 8, b[it]);
+        if (br.bias) {
+          float c[8];
+          load8(br.bias + (int64_t)m * width + (int64_t)i * 8, c);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) b[it][j] += c[j];
+        }
+#pragma unroll
+        for (int j = 0; j < 8; ++j) ss = add_square(ss, b[it][j]);
+      }
+    }
+    const float f = 1.f / sqrtf(block_sum(ss, red) / (float)width + br.eps[m]);
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+      const int i = it * 256 + threadIdx.x;
+      if (i < n8) {
+        float c[8];
+        load8(br.w + (int64_t)m * width + (int64_t)i * 8, c);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[it][j] += b[it][j] * f * c[j];
+      }
+    }
+  }
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int i = it * 256 + threadIdx.x;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[it][j] = __builtin_fmaf(v[it][j], br.scale, t[it][j]);
+    if (i < n8) {
+      if (stream) store8(stream + r * ld_s + (int64_t)i * 8, v[it]);
+      else store8(out + r * width + (int64_t)i * 8, v[it]);
+    }
+  }
+  if (!stream || !out) return;
+  group_norm_pieces<S, ITERS>(v, w, out + r * width, n8, groups, eps, sums, inv);
+}
+
+template <class SX, class SO>
+void launch_group_regs(const void* x, int64_t ld_x, void* stream_, int64_t ld_s, const int32_t* rows, const float* w, void* out,
+                       float eps, int64_t n_rows, int width, int groups, hipStream_t stream) {
+#define GN(IT)                                                                                                        \
+  group_rmsnorm_regs_kernel<SX, SO, IT><<<(unsigned)n_rows, 256, 0, stream>>>((const SX*)x, ld_x, (float*)stream_, ld_s, \
+                                                                              rows, w, (SO*)out, eps, width, groups)
+  if (width <= 256 * 8) GN(1);
+  else if (width <= 256 * 8 * 2) GN(2);
+  else GN(4);
+#undef GN
+}
+
+template <class S>
+void launch_joined_regs(const void* x, int64_t ld_x, const Branches& br, void* stream_, int64_t ld_s, const float* w,
+                        void* out, float eps, int64_t n_rows, int width, int groups, hipStream_t stream) {
+#define JN(IT)                                                                                                       \
+  joined_norms_regs_kernel<S, IT><<<(unsigned)n_rows, 256, 0, stream>>>((const S*)x, ld_x, br, (float*)stream_, ld_s, w, \
+                                                                        (S*)out, eps, width, groups)
+  if (width <= 256 * 8) JN(1);
+  else if (width <= 256 * 8 * 2) JN(2);
+  else JN(4);
+#undef JN
+}
+
+}  // namespace
+
+// x [*, ld_x]; stream (may be null) [*, ld_s], updated in place; rows (may be null) lists the source rows; w [width]
+// float; out dense [n_rows, width]. Width up to 16,384, `groups` a divisor of it.
+extern "C" int dinfer_group_rmsnorm(const void* x, int x_dtype, int64_t ld_x, void* stream_, int stream_dtype, int64_t ld_s,
+                                    const int32_t* rows, const float* w, void* out, int out_dtype, float eps,
+                                    int64_t n_rows, int64_t width, int groups, hipStream_t stream) {
+  if (n_rows <= 0) return OK;
+  if (width <= 0 || ld_x < width || (stream_ && ld_s < width) || !w || !out || groups <= 0 || width % groups ||
+      n_rows > 0x7fffffff)
+    return ERR_BAD_SHAPE;
+  for (int dt : {x_dtype, stream_dtype, out_dtype})
+    if (dt != DT_F32 && dt != DT_BF16) return ERR_BAD_DTYPE;
+  if (width > 16384 || groups > MAX_GROUPS) return ERR_UNSUPPORTED;
+  if ((!stream_ || stream_dtype == DT_F32) && width % 8 == 0 && (width / groups) % 8 == 0 && width <= 256 * 8 * 4 &&
+      ld_x % 8 == 0 && (!stream_ || (ld_s % 4 == 0 && aligned16(stream_))) && aligned16(x) && aligned16(w) && aligned16(out)) {
+    if (x_dtype == DT_F32 && out_dtype == DT_F32)
+      launch_group_regs<float, float>(x, ld_x, stream_, ld_s, rows, w, out, eps, n_rows, (int)width, groups, stream);
+    else if (x_dtype == DT_F32)
+      launch_group_regs<float, bf16>(x, ld_x, stream_, ld_s, rows, w, out, eps, n_rows, (int)width, groups, stream);
+    else if (out_dtype == DT_F32)
+      launch_group_regs<bf16, float>(x, ld_x, stream_, ld_s, rows, w, out, eps, n_rows, (int)width, groups, stream);
+    else
+      launch_group_regs<bf16, bf16>(x, ld_x, stream_, ld_s, rows, w, out, eps, n_rows, (int)width, groups, stream);
+    return launch_status();
+  }
+  // (16,384 columns and their parts' inverses: up to 68 KB of LDS, more than a launch may ask for without saying so)
+  const size_t lds = (size_t)(width + groups) * sizeof(float);
+  if (lds > 65536 && hipFuncSetAttribute((const void*)group_rmsnorm_kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                         (int)lds) != hipSuccess)
+    return ERR_LAUNCH;
+  group_rmsnorm_kernel<<<(unsigned)n_rows, 256, lds, stream>>>(
+      x, x_dtype, ld_x, stream_, stream_dtype, ld_s, rows, w, out, out_dtype, eps, (int)width, groups);
+  return launch_status();
+}
+
+// x [*, ld_x] holds `branches` rows of `width` side by side, `branch_stride` columns apart, in the step's dtype like out; bw and bias (bias may be null)
+// [branches][width] float. stream (may be null) [*, ld_s] float: then it takes the sum, and out (may be null) its group
+// norm by w; without a stream out takes the sum. Width up to 16,384.
+extern "C" int dinfer_joined_norms(int dtype, const void* x, int64_t ld_x, int branches, int64_t branch_stride, const float* bw, const float* bias,
+                                   const float* branch_eps, float scale, float* stream_, int64_t ld_s, const float* w,
+                                   void* out, float eps, int64_t n_rows, int64_t width, int groups, hipStream_t stream) {
+  if (n_rows <= 0) return OK;
+  if (width <= 0 || branches <= 0 || branch_stride < width || ld_x < branch_stride * (branches - 1) + width || (stream_ && ld_s < width) || !bw || !branch_eps ||
+      (!stream_ && !out) || (stream_ && out && !w) || groups <= 0 || width % groups || n_rows > 0x7fffffff)
+    return ERR_BAD_SHAPE;
+  if (dtype != DT_F32 && dtype != DT_BF16) return ERR_BAD_DTYPE;
+  if (width > 16384 || groups > MAX_GROUPS || branches > MAX_BRANCHES) return ERR_UNSUPPORTED;
+  Branches br{};
+  br.w = bw; br.bias = bias; br.m = branches; br.stride = branch_stride; br.scale = scale;
+  for (int m = 0; m < branches; ++m) br.eps[m] = branch_eps[m];      // (a host array)
+  if (width % 8 == 0 && (width / groups) % 8 == 0 && width <= 256 * 8 * 4 && ld_x % 8 == 0 && branch_stride % 8 == 0 &&
+      aligned16(x) && aligned16(bw) &&
+      (!bias || aligned16(bias)) && (!stream_ || (ld_s % 4 == 0 && aligned16(stream_))) && (!out || aligned16(out)) &&
+      (!w || aligned16(w))) {
+    if (dtype == DT_BF16) launch_joined_regs<bf16>(x, ld_x, br, stream_, ld_s, w, out, eps, n_rows, (int)width, groups, stream);
+    else launch_joined_regs<float>(x, ld_x, br, stream_, ld_s, w, out, eps, n_rows, (int)width, groups, stream);
+    return launch_status();
+  }
+  const size_t lds = (size_t)(width + groups) * sizeof(float);
+  DINFER_DISPATCH_DTYPE(dtype, {
+    if (lds > 65536 && hipFuncSetAttribute((const void*)joined_norms_kernel<S>, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                           (int)lds) != hipSuccess)
+      return ERR_LAUNCH;
+    joined_norms_kernel<S><<<(unsigned)n_rows, 256, lds, stream>>>((const S*)x, ld_x, br, stream_, ld_s, w, (S*)out, eps,
+                                                                  (int)width, groups);
+  });
+  return launch_status();
+}

@@ -32,6 +32,18 @@ namespace {
 constexpr int MAX_D = 512;
 constexpr int WAVES = 4;
 
+// Values mixed with another row's: v <- (1 - share) v + share first[t], `first` [T, ld] in the step's dtype, its kv heads
+// side by side as v's are (null: v stays as it is).
+struct ValueMix {
+  const void* first;
+  int64_t ld;
+  float share;
+};
+template <class S>
+__device__ __forceinline__ float mixed_value(float v, const ValueMix& mix, int64_t t, int c) {
+  return __builtin_fmaf(mix.share, to_f32(((const S*)mix.first)[t * mix.ld + c]), (1.f - mix.share) * v);
+}
+
 __device__ __forceinline__ bf16x8 zero8() {
   bf16x8 z;
 #pragma unroll
@@ -45,7 +57,7 @@ __global__ void __launch_bounds__(WAVES * 64) qkv_post_kernel(
     const void* __restrict__ wk, int wf32, float eps, float w_offset, const int32_t* __restrict__ pos,
     const float* __restrict__ cos_sin, int rot, int style, S* __restrict__ k_cache, S* __restrict__ v_cache,
     const int64_t* __restrict__ slots, int H, int Hkv, int D, int page, int Dv, const float* __restrict__ bias,
-    float temp_coef, int temp_every, const float* __restrict__ head_scale) {
+    float temp_coef, int temp_every, const float* __restrict__ head_scale, ValueMix mix) {
   __shared__ float xs[WAVES][MAX_D];
   const int64_t t = blockIdx.x;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -63,9 +75,13 @@ __global__ void __launch_bounds__(WAVES * 64) qkv_post_kernel(
     const int hk = item - H - Hkv;
     const S* vs = row + v_off + (int64_t)hk * Dv;
     S* vd = v_cache + ((blk * Hkv + hk) * (int64_t)Dv) * page + off;
-    if (bias) {
-      const float* vb = bias + (int64_t)(H + Hkv) * D + (int64_t)hk * Dv;
-      for (int d = lane; d < Dv; d += 64) vd[(int64_t)d * page] = from_f32<S>(to_f32(vs[d]) + vb[d]);
+    if (bias || mix.first) {
+      const float* vb = bias ? bias + (int64_t)(H + Hkv) * D + (int64_t)hk * Dv : nullptr;
+      for (int d = lane; d < Dv; d += 64) {
+        float v = to_f32(vs[d]) + (vb ? vb[d] : 0.f);
+        if (mix.first) v = mixed_value<S>(v, mix, t, hk * Dv + d);
+        vd[(int64_t)d * page] = from_f32<S>(v);
+      }
     } else {
       for (int d = lane; d < Dv; d += 64) vd[(int64_t)d * page] = vs[d];
     }
@@ -239,7 +255,7 @@ __global__ void __launch_bounds__(WAVES * 64) qkv_post_neox_kernel(
 __device__ __forceinline__ void v_write_transposed(const bf16* __restrict__ qkv, int64_t ld, int64_t v_off,
                                                    bf16* __restrict__ v_cache, const int64_t* __restrict__ slots, int T,
                                                    int Hkv, int D, int page, int group, int hk,
-                                                   const float* __restrict__ vb = nullptr) {
+                                                   const float* __restrict__ vb = nullptr, ValueMix mix = ValueMix{}) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int t0 = (group * WAVES + wave) * 8;
   if (t0 >= T) return;
@@ -260,6 +276,14 @@ __device__ __forceinline__ void v_write_transposed(const bf16* __restrict__ qkv,
         if (j < n) {
           v[j][0] = (bf16)((float)v[j][0] + b0);
           v[j][1] = (bf16)((float)v[j][1] + b1);
+        }
+    }
+    if (mix.first) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        if (j < n) {
+          v[j][0] = (bf16)mixed_value<bf16>((float)v[j][0], mix, t0 + j, hk * D + 2 * d2);
+          v[j][1] = (bf16)mixed_value<bf16>((float)v[j][1], mix, t0 + j, hk * D + 2 * d2 + 1);
         }
     }
     if (aligned) {
@@ -301,13 +325,13 @@ __global__ void __launch_bounds__(WAVES * 64) qkv_post_vec_kernel(
     const void* __restrict__ wk, int wf32, float eps, float w_offset, const int32_t* __restrict__ pos,
     const float* __restrict__ cos_sin, bf16* __restrict__ k_cache, bf16* __restrict__ v_cache,
     const int64_t* __restrict__ slots, int H, int Hkv, int page, int tokens, int gather_v,
-    const float* __restrict__ bias, float temp_coef, int temp_every, const float* __restrict__ head_scale) {
+    const float* __restrict__ bias, float temp_coef, int temp_every, const float* __restrict__ head_scale, ValueMix mix) {
   constexpr int D = LPH * 8, HALF = D / 2, HPW = 64 / LPH;  // heads per wave
   if ((int)blockIdx.x >= tokens) {
     const int j = (int)blockIdx.x - tokens;
     if (blockIdx.y == 0)
       v_write_transposed(qkv, ld, v_off, v_cache, slots, tokens, Hkv, D, page, j / Hkv, j % Hkv,
-                         bias ? bias + (int64_t)(H + Hkv + j % Hkv) * D : nullptr);
+                         bias ? bias + (int64_t)(H + Hkv + j % Hkv) * D : nullptr, mix);
     return;
   }
   const bool skip_v = gather_v > 0;
@@ -379,6 +403,11 @@ __global__ void __launch_bounds__(WAVES * 64) qkv_post_vec_kernel(
     }
     if (is_v) {
       if (slot >= 0 && !skip_v) {
+        if (mix.first) {
+          const bf16x8 f = *(const bf16x8*)((const bf16*)mix.first + t * mix.ld + (int64_t)(item - H - Hkv) * D + d0);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[e] = __builtin_fmaf(mix.share, (float)f[e], (1.f - mix.share) * x[e]);
+        }
         bf16* vd = v_cache + ((blk * Hkv + (item - H - Hkv)) * (int64_t)D + d0) * page + off;
 #pragma unroll
         for (int e = 0; e < 8; ++e) vd[(int64_t)e * page] = (bf16)x[e];
@@ -429,7 +458,148 @@ __global__ void __launch_bounds__(WAVES * 64) qkv_post_vec_kernel(
   }
 }
 
+// Norms over the whole projection: all q heads of a token share one root mean square, all k heads another (gains
+// [H D] and [Hkv D], float), before the rotation. A workgroup takes a token: the row waits in LDS as floats between the
+// sums and the rotation, which reads a pair's other element there. P: entries a thread takes at a time (8: bf16 rows of
+// whole 16-byte pieces that no boundary of a head, of its rotated part or of that part's halves cuts; else 1).
+// gather_v as in qkv_post_vec_kernel (P = 8 only).
+template <class S, int P>
+__global__ void __launch_bounds__(256) qkv_row_post_kernel(
+    S* __restrict__ qkv, int64_t ld, int64_t q_off, int64_t k_off, int64_t v_off, const float* __restrict__ wq,
+    const float* __restrict__ wk, float eps, const int32_t* __restrict__ pos, const float* __restrict__ cos_sin, int rot,
+    int style, S* __restrict__ k_cache, S* __restrict__ v_cache, const int64_t* __restrict__ slots, int H, int Hkv, int D,
+    int page, int Dv, const float* __restrict__ bias, int tokens, int gather_v, ValueMix mix) {
+  extern __shared__ __attribute__((aligned(16))) float row_smem[];
+  __shared__ float red[16];
+  if constexpr (P == 8) {
+    if ((int)blockIdx.x >= tokens) {
+      const int j = (int)blockIdx.x - tokens;
+      v_write_transposed((const bf16*)qkv, ld, v_off, (bf16*)v_cache, slots, tokens, Hkv, Dv, page, j / Hkv, j % Hkv,
+                         bias ? bias + (int64_t)(H + Hkv) * D + (int64_t)(j % Hkv) * Dv : nullptr, mix);
+      return;
+    }
+  }
+  const int64_t t = blockIdx.x;
+  S* row = qkv + t * ld;
+  const int64_t slot = slots ? slots[t] : -1;
+  const int64_t blk = slot >= 0 ? slot / page : 0;
+  const int off = slot >= 0 ? (int)(slot % page) : 0;
+  const int nq = H * D, n = nq + Hkv * D;
+  float sq = 0.f, sk = 0.f;
+  for (int i = threadIdx.x * P; i < n; i += 256 * P) {
+    const S* src = i < nq ? row + q_off + i : row + k_off + (i - nq);
+    float v[P];
+    if constexpr (P == 8) {
+      const bf16x8 x = *(const bf16x8*)src;
+#pragma unroll
+      for (int e = 0; e < P; ++e) v[e] = (float)x[e];
+    } else {
+      v[0] = to_f32(src[0]);
+    }
+#pragma unroll
+    for (int e = 0; e < P; ++e) {
+      if (bias) v[e] += bias[i + e];
+      row_smem[i + e] = v[e];
+      if (i < nq) sq = add_square(sq, v[e]);
+      else sk = add_square(sk, v[e]);
+    }
+  }
+  // (the barriers inside also publish the row)
+  const float fq = 1.f / sqrtf(block_sum(sq, red) / (float)nq + eps);
+  const float fk = 1.f / sqrtf(block_sum(sk, red) / (float)(n - nq) + eps);
+  const float* cs = cos_sin ? cos_sin + (int64_t)pos[t] * rot : nullptr;
+  const int half = rot / 2, Dp = (D + 7) & ~7;
+  for (int i = threadIdx.x * P; i < n; i += 256 * P) {
+    const bool is_q = i < nq;
+    const int e0 = is_q ? i : i - nq, hd = e0 / D, d = e0 - hd * D;
+    const float* w = is_q ? wq : wk;
+    const float f = is_q ? fq : fk;
+    float y[P];
+#pragma unroll
+    for (int e = 0; e < P; ++e) y[e] = row_smem[i + e] * f * w[e0 + e];
+    if (cs && d < rot) {
+      float r[P];
+#pragma unroll
+      for (int e = 0; e < P; ++e) {
+        const int de = d + e;
+        const bool first = style == 0 ? de < half : (de & 1) == 0;
+        const int pi = style == 0 ? (first ? de : de - half) : de >> 1;
+        const int step = style == 0 ? half : 1, other = first ? step : -step;
+        const float o = row_smem[i + e + other] * f * w[e0 + e + other];
+        r[e] = first ? rotated_first(y[e], o, cs[pi], cs[half + pi]) : rotated_second(o, y[e], cs[pi], cs[half + pi]);
+      }
+#pragma unroll
+      for (int e = 0; e < P; ++e) y[e] = r[e];
+    }
+    S* to = is_q ? row + q_off + e0
+                 : !slots ? row + k_off + e0
+                          : slot >= 0 ? k_cache + (blk * Hkv + hd) * (int64_t)page * Dp + k_page_offset(off, d, page) : nullptr;
+    if (!to) continue;
+    if constexpr (P == 8) {
+      bf16x8 r;
+#pragma unroll
+      for (int e = 0; e < P; ++e) r[e] = (bf16)y[e];
+      *(bf16x8*)to = r;
+    } else {
+      to[0] = from_f32<S>(y[0]);
+    }
+  }
+  if (slot < 0 || !v_cache || gather_v > 0) return;
+  for (int i = threadIdx.x; i < Hkv * Dv; i += 256) {
+    float v = to_f32(row[v_off + i]);
+    if (bias) v += bias[n + i];
+    if (mix.first) v = mixed_value<S>(v, mix, t, i);
+    v_cache[(blk * Hkv * Dv + i) * (int64_t)page + off] = from_f32<S>(v);
+  }
+}
+
 }  // namespace
+
+// qkv_post with norms over the whole projection: q_gain [heads head_dim], k_gain [kv_heads head_dim], float. Everything
+// else as there.
+extern "C" int dinfer_qkv_row_post(int dtype, void* qkv, int64_t tokens, int64_t ld, int64_t q_off, int64_t k_off,
+                                   int64_t v_off, const float* q_gain, const float* k_gain, float eps,
+                                   const int32_t* positions, const float* cos_sin, int rotary_dim, int style, void* k_cache,
+                                   void* v_cache, const int64_t* slot_mapping, int heads, int kv_heads, int head_dim,
+                                   int page_size, int token_runs, int v_dim, const float* bias, const void* v_first,
+                                   int64_t ld_v_first, float v_share, hipStream_t stream) {
+  if (v_dim <= 0) v_dim = head_dim;
+  if (tokens <= 0) return OK;
+  if (heads <= 0 || kv_heads <= 0 || head_dim <= 0 || page_size <= 0 || tokens > 0x7fffffff || !q_gain || !k_gain)
+    return ERR_BAD_SHAPE;
+  if (cos_sin && (rotary_dim <= 0 || rotary_dim > head_dim || rotary_dim % 2 != 0)) return ERR_BAD_SHAPE;
+  if (style != 0 && style != 1) return ERR_UNSUPPORTED;
+  const int64_t n = (int64_t)(heads + kv_heads) * head_dim;
+  if (n > 32768) return ERR_UNSUPPORTED;      // (128 KB of LDS)
+  const size_t lds = (size_t)n * sizeof(float);
+  const ValueMix mix{v_first, ld_v_first, v_share};
+  const int rot = cos_sin ? rotary_dim : 0;
+  const bool vec = dtype == DT_BF16 && head_dim % 8 == 0 && rot % (style == 0 ? 16 : 8) == 0 && ld % 8 == 0 && q_off % 8 == 0 &&
+                   k_off % 8 == 0 && v_off % 2 == 0 && v_dim % 2 == 0 && ((uintptr_t)qkv % 16) == 0 &&
+                   ((uintptr_t)k_cache % 16) == 0;
+  if (vec) {
+    const bool gather = slot_mapping && v_cache && token_runs && tokens >= 64 && page_size % 8 == 0 &&
+                        ((uintptr_t)v_cache % 16) == 0;
+    const int64_t gather_v = gather ? (tokens + 8 * WAVES - 1) / (8 * WAVES) * kv_heads : 0;
+    if (tokens + gather_v > 0x7fffffff) return ERR_BAD_SHAPE;
+    auto kernel = qkv_row_post_kernel<bf16, 8>;
+    if (lds > 65536 - 64 && hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
+      return ERR_LAUNCH;
+    kernel<<<(unsigned)(tokens + gather_v), 256, lds, stream>>>(
+        (bf16*)qkv, ld, q_off, k_off, v_off, q_gain, k_gain, eps, positions, cos_sin, rot, style, (bf16*)k_cache, (bf16*)v_cache,
+        slot_mapping, heads, kv_heads, head_dim, page_size, v_dim, bias, (int)tokens, (int)gather_v, mix);
+    return launch_status();
+  }
+  DINFER_DISPATCH_DTYPE(dtype, {
+    auto kernel = qkv_row_post_kernel<S, 1>;
+    if (lds > 65536 - 64 && hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
+      return ERR_LAUNCH;
+    kernel<<<(unsigned)tokens, 256, lds, stream>>>((S*)qkv, ld, q_off, k_off, v_off, q_gain, k_gain, eps, positions, cos_sin, rot,
+                                                   style, (S*)k_cache, (S*)v_cache, slot_mapping, heads, kv_heads, head_dim,
+                                                   page_size, v_dim, bias, (int)tokens, 0, mix);
+  });
+  return launch_status();
+}
 
 extern "C" int dinfer_qkv_post(int dtype, void* qkv, int64_t tokens, int64_t ld, int64_t q_off, int64_t k_off,
                                int64_t v_off, const void* q_gain, const void* k_gain, int w_f32, float eps,
@@ -437,7 +607,9 @@ extern "C" int dinfer_qkv_post(int dtype, void* qkv, int64_t tokens, int64_t ld,
                                int style, void* k_cache, void* v_cache, const int64_t* slot_mapping, int heads,
                                int kv_heads, int head_dim, int page_size, int token_runs, int v_dim,
                                const float* bias, float temp_coef, int temp_every, const float* head_scale,
-                               hipStream_t stream) {
+                               const void* v_first, int64_t ld_v_first, float v_share, hipStream_t stream) {
+  // v_first (may be null): [tokens, ld_v_first] in the step's dtype, kv heads of v_dim side by side; the cached values are
+  // (1 - v_share) v + v_share v_first.
   // head_scale (may be null): float [heads], q of head h is multiplied by head_scale[h] with the norm (gains needed).
   // bias (may be null): float [q heads | k heads | v heads], added to the product's output before anything else.
   // temp_every > 0: q is multiplied by 1 + temp_coef ln(floor((p + 1) / temp_every) + 1) with the norm (gains needed).
@@ -456,11 +628,13 @@ extern "C" int dinfer_qkv_post(int dtype, void* qkv, int64_t tokens, int64_t ld,
   if ((temp_every > 0 || head_scale) && !q_gain) return ERR_UNSUPPORTED;
   const bool whole_head_neox = style == 0 && head_dim % 8 == 0 && (!cos_sin || rotary_dim == head_dim) &&
                                v_dim == head_dim && (v_cache || !slot_mapping);
-  const bool plain_head = !bias && temp_every <= 0 && !head_scale;   // what the kernels of 2-byte accesses for whole heads take
+  const ValueMix mix{v_first, ld_v_first, v_share};
+  const bool plain_head = !bias && temp_every <= 0 && !head_scale && !v_first;   // what the kernels of 2-byte accesses for whole heads take
   const bool vec_ok = dtype == DT_BF16 && (head_dim == 64 || head_dim == 128 || head_dim == 256) && ld % 8 == 0 &&
                       q_off % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && ((uintptr_t)qkv % 16) == 0 &&
                       ((uintptr_t)q_gain % 16) == 0 && ((uintptr_t)k_gain % 16) == 0 && ((uintptr_t)cos_sin % 16) == 0 &&
-                      ((uintptr_t)k_cache % 16) == 0 && ((uintptr_t)bias % 16) == 0;
+                      ((uintptr_t)k_cache % 16) == 0 && ((uintptr_t)bias % 16) == 0 &&
+                      (!v_first || (((uintptr_t)v_first % 16) == 0 && ld_v_first % 8 == 0));
   if (whole_head_neox && vec_ok) {
     const int lph = head_dim / 8, hpw = 64 / lph;
     // many tokens fill the chip with one workgroup each; few tokens spread their heads over several
@@ -474,7 +648,7 @@ extern "C" int dinfer_qkv_post(int dtype, void* qkv, int64_t tokens, int64_t ld,
   qkv_post_vec_kernel<LPH_><<<vgrid, WAVES * 64, 0, stream>>>(                                                         \
       (bf16*)qkv, ld, q_off, k_off, v_off, q_gain, k_gain, w_f32, eps, w_offset, positions, cos_sin, (bf16*)k_cache, \
       (bf16*)v_cache, slot_mapping, heads, kv_heads, page_size, (int)tokens, (int)gather_v, bias, temp_coef,       \
-      temp_every, head_scale)
+      temp_every, head_scale, mix)
     if (lph == 8) DINFER_QKV_VEC(8);
     else if (lph == 16) DINFER_QKV_VEC(16);
     else DINFER_QKV_VEC(32);
@@ -504,7 +678,7 @@ extern "C" int dinfer_qkv_post(int dtype, void* qkv, int64_t tokens, int64_t ld,
                                                         w_offset, positions, cos_sin, rotary_dim, style, (S*)k_cache,
                                                         (S*)v_cache, slot_mapping, heads, kv_heads, head_dim,
                                                         page_size, v_dim, bias, temp_coef, temp_every,
-                                                        head_scale);
+                                                        head_scale, mix);
   });
   return launch_status();
 }

@@ -250,6 +250,52 @@ def rmsnorm_stream(stream: torch.Tensor, n_rows: int, *, branch: torch.Tensor | 
     return out
 
 
+def group_rmsnorm(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, eps: float, n_rows: int, groups: int, *,
+                  residual: torch.Tensor | None = None, rows: torch.Tensor | None = None) -> torch.Tensor:
+    """out[r] = x[src r] with each of `groups` equal consecutive parts of the row divided by its own root mean square (eps
+    inside the root), times weight (float32). residual: updated in place to round(x + residual) in its own type first, and
+    that sum is normed. rows: int32 indices of the n_rows source rows. x, residual and out may each be float32 or bfloat16."""
+    _need_gpu(x, weight, out, residual, rows)
+    width = out.shape[1]
+    assert x.shape[1] == width and weight.numel() == width and weight.is_contiguous() and weight.dtype == torch.float32
+    assert out.is_contiguous() and out.shape[0] >= n_rows and width % groups == 0
+    if rows is None:
+        assert x.shape[0] >= n_rows
+    else:
+        assert rows.dtype == torch.int32 and rows.is_contiguous() and rows.numel() >= n_rows
+    if residual is not None:
+        assert residual.shape == x.shape
+    lib.call("dinfer_group_rmsnorm", x.data_ptr(), dtype_code(x.dtype), _rows(x), _ptr(residual),
+             dtype_code(residual.dtype) if residual is not None else 0, _rows(residual) if residual is not None else 0,
+             _ptr(rows), weight.data_ptr(), out.data_ptr(), dtype_code(out.dtype), float(eps), n_rows, width, int(groups),
+             _stream())
+    return out
+
+
+JOINED_NORMS_MAX = 4     # branches one row may hold
+
+
+def joined_norms(x: torch.Tensor, weights: torch.Tensor, n_rows: int, *, eps: list, scale: float,
+                 bias: torch.Tensor | None = None, stream: torch.Tensor | None = None, out: torch.Tensor | None = None,
+                 weight: torch.Tensor | None = None, norm_eps: float = 0.0, groups: int = 1) -> None:
+    """x [T, M * stride]: M branches of `width` columns side by side (stride: width rounded up to 8). y = scale * sum_m rms_m(x_m + bias[m]) * weights[m], each branch normed
+    over its own width with eps[m]. Without a stream y goes to out; with one (float32) stream += y in place and out, where
+    given, takes the group norm (weight, norm_eps, groups) of the new stream. weights, bias [M, width], weight: float32."""
+    _need_gpu(x, weights, bias, stream, out, weight)
+    M, width = weights.shape
+    assert weights.dtype == torch.float32 and weights.is_contiguous() and len(eps) == M
+    stride = -(-width // 8) * 8
+    assert x.shape[1] == M * stride
+    assert x.shape[0] >= n_rows and (bias is None or (bias.dtype == torch.float32 and bias.shape == weights.shape and bias.is_contiguous()))
+    assert stream is None or (stream.dtype == torch.float32 and stream.shape[1] == width and stream.shape[0] >= n_rows)
+    assert out is None or (out.dtype == x.dtype and out.is_contiguous() and out.shape[1] == width and out.shape[0] >= n_rows)
+    assert weight is None or (weight.dtype == torch.float32 and weight.numel() == width and weight.is_contiguous())
+    branch_eps = (ctypes.c_float * M)(*eps)      # (read by the launcher before it returns)
+    lib.call("dinfer_joined_norms", dtype_code(x.dtype), x.data_ptr(), _rows(x), M, stride, weights.data_ptr(), _ptr(bias),
+             ctypes.addressof(branch_eps), float(scale), _ptr(stream), _rows(stream) if stream is not None else 0,
+             _ptr(weight), _ptr(out), float(norm_eps), n_rows, width, int(groups), _stream())
+
+
 def axpby(a: torch.Tensor, alpha: float, b: torch.Tensor, beta: float, out: torch.Tensor, rows: int) -> torch.Tensor:
     """out[:rows] = alpha * a[:rows] + beta * b[:rows]; out may be a or b."""
     _need_gpu(a, b, out)
@@ -493,6 +539,83 @@ def gated_group_norm(y: torch.Tensor, z: torch.Tensor, z_off: int, out: torch.Te
     return out
 
 
+# ---- gated linear attention -------------------------------------------------------------------------
+GLA_MAX_DIM = 256        # the largest key size of the recurrence kernel
+GLA_MAX_LOW = 512        # the largest inner size of the decay projection
+
+
+def channel_decay(proj: torch.Tensor, tokens: int, *, low_off: int, w2t: torch.Tensor, bias: torch.Tensor, tau: float,
+                  out: torch.Tensor) -> torch.Tensor:
+    """out[t, c] = sigmoid(sum_r w2t[r, c] proj[t, low_off + r] + bias[c])^(1 / tau), float32. w2t [low, C] (the second
+    factor of the decay projection, transposed) and bias [C] float32."""
+    _need_gpu(proj, w2t, bias, out)
+    low, C = w2t.shape
+    assert w2t.dtype == bias.dtype == out.dtype == torch.float32 and w2t.is_contiguous() and bias.numel() == C
+    assert proj.shape[0] >= tokens and out.shape[0] >= tokens and out.shape[1] >= C and low_off + low <= proj.shape[1]
+    lib.call("dinfer_channel_decay", dtype_code(proj.dtype), proj.data_ptr(), _rows(proj), low_off, low, w2t.data_ptr(),
+             bias.data_ptr(), 1.0 / float(tau), out.data_ptr(), _rows(out), tokens, C, _stream())
+    return out
+
+
+def gla_places(tokens: int, reqs: int) -> int:
+    """Chunks whose notes gla_recurrence may keep in a step of up to that many tokens and requests."""
+    return tokens // int(lib.get("dinfer_gla_chunk")()) + reqs + 1
+
+
+def gla_cuts(tokens: int, max_rows: int, num_reqs: int, heads: int, vdim: int) -> bool:
+    """Whether a step of these counts runs in chunks side by side (a rule of the counts alone)."""
+    return bool(lib.get("dinfer_gla_cuts")(tokens, max_rows, num_reqs, heads, vdim))
+
+
+def gla_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, state: torch.Tensor,
+                   out: torch.Tensor, *, q_scale: float, notes: torch.Tensor | None, products: torch.Tensor | None,
+                   state_slots: torch.Tensor, cu_seqlens: torch.Tensor, seq_lens: torch.Tensor, num_reqs: int, tokens: int,
+                   max_rows: int, cut: bool, heads: int, dim: int, vdim: int) -> torch.Tensor:
+    """Per request and head, token by token: S <- diag(decay) S + k v^T, out = S^T (q * q_scale). q, k [T, heads dim] and v
+    [T, heads vdim] are column blocks of one buffer as the projections left them; decay float32 [T, heads dim]. state
+    [slots, heads, vdim, dim] float32, updated in place; out [T, heads vdim] float32. cut: in chunks side by side, with
+    scratch notes [places, heads, vdim, dim] and products [places, heads, dim] (gla_places of the step at least)."""
+    _need_gpu(q, k, v, decay, state, out, notes, products, state_slots, cu_seqlens, seq_lens)
+    assert q.dtype == k.dtype == v.dtype and _rows(q) == _rows(k) == _rows(v)
+    assert decay.dtype == state.dtype == out.dtype == torch.float32 and state.is_contiguous()
+    assert tuple(state.shape[1:]) == (heads, vdim, dim) and out.shape[1] >= heads * vdim and decay.shape[1] >= heads * dim
+    assert q.shape[1] >= heads * dim and k.shape[1] >= heads * dim and v.shape[1] >= heads * vdim
+    assert min(t.shape[0] for t in (q, k, v, decay, out)) >= tokens
+    places = 0
+    if cut:
+        assert notes is not None and notes.dtype == products.dtype == torch.float32
+        assert notes.is_contiguous() and products.is_contiguous()
+        places = min(notes.numel() // (heads * vdim * dim), products.numel() // (heads * dim))
+    lib.call("dinfer_gla_recurrence", dtype_code(q.dtype), q.data_ptr(), k.data_ptr(), v.data_ptr(), _rows(q),
+             decay.data_ptr(), _rows(decay), float(q_scale), state.data_ptr(), _ptr(notes) if cut else 0,
+             _ptr(products) if cut else 0, places, state_slots.data_ptr(), cu_seqlens.data_ptr(), seq_lens.data_ptr(),
+             out.data_ptr(), _rows(out), num_reqs, tokens, max_rows, int(cut), heads, dim, vdim, _stream())
+    return out
+
+
+# ---- gated recurrence of single channels ---------------------------------------------------------------
+def min_gru_places(tokens: int, reqs: int) -> int:
+    """Chunks whose notes min_gru may keep in a step of up to that many tokens and requests."""
+    return tokens // int(lib.get("dinfer_min_gru_chunk")()) + reqs + 1
+
+
+def min_gru(proj: torch.Tensor, out: torch.Tensor, *, z_off: int, x_off: int, g_off: int, z_bias: torch.Tensor,
+            x_bias: torch.Tensor, state: torch.Tensor, notes: torch.Tensor, state_slots: torch.Tensor,
+            cu_seqlens: torch.Tensor, seq_lens: torch.Tensor, num_reqs: int, tokens: int, max_rows: int) -> torch.Tensor:
+    """a = sigmoid(z + z_bias), u = x + x_bias, c = u + 1/2 (u >= 0) or sigmoid(u); S <- (1 - a) S + a c per channel and
+    token; out = S * silu(g). state [slots, N] float32, updated in place; notes float32 scratch of min_gru_places * 2 N."""
+    _need_gpu(proj, out, z_bias, x_bias, state, notes, state_slots, cu_seqlens, seq_lens)
+    N = state.shape[1]
+    assert state.dtype == z_bias.dtype == x_bias.dtype == notes.dtype == torch.float32
+    assert state.is_contiguous() and notes.is_contiguous() and z_bias.numel() == N == x_bias.numel()
+    assert proj.dtype == out.dtype and max(z_off, x_off, g_off) + N <= proj.shape[1] and out.shape[1] >= N
+    assert proj.shape[0] >= tokens and out.shape[0] >= tokens
+    lib.call("dinfer_min_gru", dtype_code(proj.dtype), proj.data_ptr(), _rows(proj), z_off, x_off, g_off, z_bias.data_ptr(),
+             x_bias.data_ptr(), state.data_ptr(), notes.data_ptr(), notes.numel() // (2 * N), state_slots.data_ptr(),
+             cu_seqlens.data_ptr(), seq_lens.data_ptr(), out.data_ptr(), _rows(out), num_reqs, tokens, max_rows, N, _stream())
+    return out
+
+
 # ---- several residual streams ----------------------------------------------------------------------
 STREAMS_MAX = 8          # streams a token the kernel holds in registers
 STREAMS_MAX_WIDTH = 12288
@@ -659,7 +782,7 @@ MOE_MAX_EXPERTS = 1024   # the routing and sorting kernels keep one number an ex
 MOE_MAX_TOP = 64         # a lane of the routing wave keeps one choice
 
 
-EXPERT_ACTS = {"silu": 2, "gelu": 3}    # activations the plain (not gated) expert products apply -> their code
+EXPERT_ACTS = {"silu": 2, "gelu": 3, "relu2": 4}    # activations the plain (not gated) expert products apply -> their code
 
 
 def moe_tile_rows(dtype: torch.dtype, entries: int, experts: int, k_in: int, k_mid: int) -> int:
@@ -675,15 +798,15 @@ def moe_max_tiles(entries: int, experts: int, tile_rows: int) -> int:
 
 def moe_route(x: torch.Tensor, router: torch.Tensor, shared_gate_w: torch.Tensor | None, idx: torch.Tensor,
               share: torch.Tensor, shared_gate: torch.Tensor | None, tokens: int, top: int, z: torch.Tensor,
-              all_scores: bool = False, correction: torch.Tensor | None = None) -> None:
+              all_scores: int = 0, correction: torch.Tensor | None = None) -> None:
     """Per token: logits x @ router.T in float (router float32 [experts, width]), idx[t] the `top` largest (lowest index
     among equals), share[t] the softmax over them; shared_gate[t] = sigmoid(x . shared_gate_w) where that is given.
-    z: float32 scratch of tokens * (experts + 1) for the logits. all_scores: the scores are the softmax over all
+    z: float32 scratch of tokens * (experts + 1) for the logits. all_scores 1: the scores are the softmax over all
     experts, the choice goes by score + correction (float32 [experts], or none) and share[t] holds the chosen scores
-    as they are."""
+    as they are; 2: the scores are the sigmoids of the logits, and share[t] holds the chosen ones."""
     _need_gpu(x, router, shared_gate_w, idx, share, shared_gate, z, correction)
     if correction is not None:
-        assert all_scores and correction.dtype == torch.float32 and correction.numel() == router.shape[0]
+        assert all_scores == 1 and correction.dtype == torch.float32 and correction.numel() == router.shape[0]
     experts, width = router.shape
     assert router.dtype == torch.float32 and router.is_contiguous() and x.shape[1] == width and x.shape[0] >= tokens
     assert idx.dtype == torch.int32 and share.dtype == torch.float32 and idx.is_contiguous() and share.is_contiguous()
@@ -714,12 +837,14 @@ def moe_scatter(idx: torch.Tensor, entries: int, experts: int, offsets: torch.Te
 
 def experts_nt(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, entries: int, tiles: torch.Tensor,
                offsets: torch.Tensor, perm: torch.Tensor, *, gated: bool, a_div: int, c_to_perm: bool,
-               tile_rows: int, act: str | None = None) -> torch.Tensor:
+               tile_rows: int, act: str | None = None, row_scale: torch.Tensor | None = None) -> torch.Tensor:
     """The products of all experts in one launch. w [experts, rows, K]; gated: rows = 2 N, gate rows first, and
     out = silu(a Wg^T) * (a Wu^T). a_div > 0: the row of sorted place i is a[perm[i] // a_div] (the step's tokens),
     0: a[i]. c_to_perm: the result of sorted place i goes to out[perm[i]], else to out[i]. tile_rows: what moe_scatter
-    made the work list with. act (not gated): "silu" or "gelu" (error function) on every result."""
-    _need_gpu(a, w, out, tiles, offsets, perm)
+    made the work list with. act (not gated): "silu", "gelu" (error function) or "relu2" on every result. row_scale: float32,
+    a factor an entry that multiplies the entry's row of a (on the float sums, before the activation)."""
+    _need_gpu(a, w, out, tiles, offsets, perm, row_scale)
+    assert row_scale is None or (row_scale.dtype == torch.float32 and row_scale.is_contiguous() and row_scale.numel() >= entries)
     if act is not None and (gated or act not in EXPERT_ACTS):
         raise lib.KernelError(f"experts: activation {act!r} has no kernel here (known: {sorted(EXPERT_ACTS)}, not gated)")
     experts, rows, k = w.shape
@@ -728,27 +853,27 @@ def experts_nt(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, entries: int
     assert out.shape[0] >= entries and (a_div > 0 or a.shape[0] >= entries)
     lib.call("dinfer_experts_nt", dtype_code(a.dtype), 1 if gated else EXPERT_ACTS[act] if act else 0, a.data_ptr(), _rows(a), w.data_ptr(), k,
              rows * k, out.data_ptr(), _rows(out), n, k, tiles.data_ptr(), moe_max_tiles(entries, experts, tile_rows),
-             int(tile_rows), offsets.data_ptr(), perm.data_ptr(), int(a_div), 1 if c_to_perm else 0, _stream())
+             int(tile_rows), offsets.data_ptr(), perm.data_ptr(), int(a_div), 1 if c_to_perm else 0, _ptr(row_scale), _stream())
     return out
 
 
-def moe_combine(y: torch.Tensor, share: torch.Tensor, top: int, shared: torch.Tensor | None,
+def moe_combine(y: torch.Tensor, share: torch.Tensor | None, top: int, shared: torch.Tensor | None,
                 shared_gate: torch.Tensor | None, out: torch.Tensor, tokens: int, idx: torch.Tensor | None = None,
                 real_experts: int = 0, x: torch.Tensor | None = None) -> torch.Tensor:
     """out[t] = sum_c share[t, c] * y[t * top + c] (+ shared_gate[t] * shared[t], or + shared[t] without a gate).
     idx, real_experts, x: a choice idx[t, c] >= real_experts stands for an expert whose output is its input: x[t] takes
-    the place of y[t * top + c]."""
+    the place of y[t * top + c]. share None: every choice counts as it is."""
     _need_gpu(y, share, shared, shared_gate, out, idx, x)
     if idx is not None:
         assert idx.dtype == torch.int32 and idx.numel() >= tokens * top and x is not None
         assert x.dtype == out.dtype and x.shape[1] >= out.shape[1] and x.shape[0] >= tokens
     width = out.shape[1]
     assert y.shape[1] == width and y.dtype == out.dtype and y.shape[0] >= tokens * top and out.shape[0] >= tokens
-    assert share.dtype == torch.float32 and share.numel() >= tokens * top
+    assert share is None or (share.dtype == torch.float32 and share.numel() >= tokens * top)
     if shared is not None:
         assert shared.dtype == out.dtype and shared.shape[1] == width and shared.shape[0] >= tokens
         assert shared_gate is None or (shared_gate.dtype == torch.float32 and shared_gate.numel() >= tokens)
-    lib.call("dinfer_moe_combine", dtype_code(y.dtype), y.data_ptr(), _rows(y), share.data_ptr(), top, _ptr(shared),
+    lib.call("dinfer_moe_combine", dtype_code(y.dtype), y.data_ptr(), _rows(y), _ptr(share), top, _ptr(shared),
              _rows(shared) if shared is not None else 0, _ptr(shared_gate), out.data_ptr(), _rows(out), tokens, width,
              _ptr(idx), int(real_experts), _ptr(x) if idx is not None else 0, _rows(x) if idx is not None else 0, _stream())
     return out
@@ -795,11 +920,14 @@ def qkv_post(qkv: torch.Tensor, tokens: int, *, heads: int, kv_heads: int, head_
              positions: torch.Tensor, cos_sin: torch.Tensor | None, rotary_dim: int, rope_style: int,
              k_cache: torch.Tensor | None, v_cache: torch.Tensor | None, slot_mapping: torch.Tensor | None,
              page_size: int, token_runs: bool = True, v_dim: int | None = None, bias: torch.Tensor | None = None,
-             q_temp: tuple | None = None, q_head_scale: torch.Tensor | None = None) -> None:
+             q_temp: tuple | None = None, q_head_scale: torch.Tensor | None = None, whole: bool = False,
+             v_first: torch.Tensor | None = None, v_share: float = 0.0) -> None:
     """Per-head q/k norm, rotation, q written back in place, k and v written to the cache pages.
     bias: float32 [q heads | k heads | v heads], added to the product's output first. q_temp (coef, every): q is
     multiplied by 1 + coef ln(floor((p + 1) / every) + 1) at position p, together with the norm. q_head_scale: float32
     [heads], q of head h is multiplied by its entry with the norm (a temperature on the head's scores).
+    whole: the norms run over the whole projection, all heads of a token at once (gains float32 [heads * head_dim] and
+    [kv_heads * head_dim]). v_first [T, kv_heads * v_dim]: the cached values are (1 - v_share) v + v_share v_first.
     v_dim: the size of a value head where it is not head_dim. v_cache None beside a k_cache: the values are not stored
     (a layer whose values are its keys reads them from the key pages).
 
@@ -814,7 +942,14 @@ def qkv_post(qkv: torch.Tensor, tokens: int, *, heads: int, kv_heads: int, head_
     assert max(q_off + heads * head_dim, k_off + kv_heads * head_dim, v_off + kv_heads * vd) <= qkv.shape[1]
     assert positions.dtype == torch.int32 and positions.numel() >= tokens
     wf32 = 0
-    if q_gain is not None:
+    if v_first is not None:
+        assert v_first.dtype == qkv.dtype and v_first.shape[0] >= tokens and v_first.shape[1] >= kv_heads * vd
+    first = (_ptr(v_first), _rows(v_first) if v_first is not None else 0, float(v_share))
+    if whole:
+        assert q_temp is None and q_head_scale is None and gain_offset == 0.0
+        assert q_gain.dtype == k_gain.dtype == torch.float32 and q_gain.is_contiguous() and k_gain.is_contiguous()
+        assert q_gain.numel() == heads * head_dim and k_gain.numel() == kv_heads * head_dim
+    elif q_gain is not None:
         assert q_gain.numel() == head_dim and k_gain is not None and k_gain.numel() == head_dim
         wf32 = _is_param_f32(q_gain, qkv.dtype)
         assert _is_param_f32(k_gain, qkv.dtype) == wf32
@@ -832,22 +967,32 @@ def qkv_post(qkv: torch.Tensor, tokens: int, *, heads: int, kv_heads: int, head_
         assert k_cache is not None
         _check_pages(k_cache, v_cache, kv_heads, head_dim, page_size, vd)
         assert k_cache.dtype == qkv.dtype and (v_cache is None or v_cache.dtype == qkv.dtype)
+    if whole:
+        lib.call("dinfer_qkv_row_post", dtype_code(qkv.dtype), qkv.data_ptr(), tokens, ld, q_off, k_off, v_off,
+                 q_gain.data_ptr(), k_gain.data_ptr(), float(eps), positions.data_ptr(), _ptr(cos_sin), rotary_dim,
+                 rope_style, _ptr(k_cache), _ptr(v_cache), _ptr(slot_mapping), heads, kv_heads, head_dim, page_size,
+                 int(token_runs), vd, _ptr(bias), *first, _stream())
+        return
     lib.call("dinfer_qkv_post", dtype_code(qkv.dtype), qkv.data_ptr(), tokens, ld, q_off, k_off, v_off,
              _ptr(q_gain), _ptr(k_gain), wf32, float(eps), float(gain_offset), positions.data_ptr(), _ptr(cos_sin),
              rotary_dim, rope_style, _ptr(k_cache), _ptr(v_cache), _ptr(slot_mapping), heads, kv_heads, head_dim,
              page_size, int(token_runs), vd, _ptr(bias), float(q_temp[0]) if q_temp else 0.0,
-             int(q_temp[1]) if q_temp else 0, _ptr(q_head_scale), _stream())
+             int(q_temp[1]) if q_temp else 0, _ptr(q_head_scale), *first, _stream())
 
 
 def attn_paged_ext(q: torch.Tensor, out: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor | None,
                    block_table: torch.Tensor, cu_seqlens: torch.Tensor, seq_lens: torch.Tensor, num_reqs: int,
                    tokens: int, *, scale: float, window: int, heads: int, kv_heads: int, head_dim: int, page_size: int,
                    v_dim: int | None = None, keep_first: int = 0, sinks: torch.Tensor | None = None,
-                   slope_exp: float = 0.0, out_scale: float = 1.0) -> torch.Tensor:
+                   slope_exp: float = 0.0, out_scale: float = 1.0,
+                   sigmoid_bias: torch.Tensor | None = None) -> torch.Tensor:
     """The plain kernel with its options: keys j < keep_first stay visible behind the window; sinks (float32 [heads])
     join the softmax's denominator; slope_exp E takes 2^(-E (h + 1) / heads) * distance off the scores; values of size
-    v_dim, or read from the key pages (v_cache None); the output times out_scale. Any storage type."""
-    _need_gpu(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, sinks)
+    v_dim, or read from the key pages (v_cache None); the output times out_scale; sigmoid_bias (float32 [heads]): the
+    weights are sigmoid(score + bias), not normalised. Any storage type."""
+    _need_gpu(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, sinks, sigmoid_bias)
+    if sigmoid_bias is not None:
+        assert sinks is None and sigmoid_bias.dtype == torch.float32 and sigmoid_bias.numel() == heads
     vd = head_dim if v_dim is None else v_dim
     _check_pages(k_cache, v_cache, kv_heads, head_dim, page_size, vd)
     assert q.dtype == out.dtype == k_cache.dtype and q.shape[0] >= tokens and out.shape[0] >= tokens
@@ -859,7 +1004,7 @@ def attn_paged_ext(q: torch.Tensor, out: torch.Tensor, k_cache: torch.Tensor, v_
     lib.call("dinfer_attn_paged_ext", dtype_code(q.dtype), q.data_ptr(), _rows(q), out.data_ptr(), _rows(out),
              k_cache.data_ptr(), _ptr(v_cache), block_table.data_ptr(), block_table.shape[1], cu_seqlens.data_ptr(),
              seq_lens.data_ptr(), num_reqs, tokens, float(scale), int(window), int(keep_first), _ptr(sinks),
-             float(slope_exp), heads, kv_heads, head_dim, vd, page_size, float(out_scale), _stream())
+             float(slope_exp), heads, kv_heads, head_dim, vd, page_size, float(out_scale), _ptr(sigmoid_bias), _stream())
     return out
 
 
@@ -923,12 +1068,16 @@ def attn_mfma_supports(head_dim: int, page_size: int, heads: int, kv_heads: int)
     return bool(lib.get("dinfer_attn_mfma_supports")(head_dim, page_size, heads, kv_heads))
 
 
-def _check_paged(q, out, k_cache, v_cache, block_table, seq_lens, num_reqs, heads, kv_heads, head_dim, page_size):
+def attn_flash_ext_supports(head_dim: int, v_dim: int, page_size: int, heads: int, kv_heads: int, sigmoid: bool = False) -> bool:
+    return bool(lib.get("dinfer_attn_flash_ext_supports")(head_dim, v_dim, page_size, heads, kv_heads, int(sigmoid)))
+
+
+def _check_paged(q, out, k_cache, v_cache, block_table, seq_lens, num_reqs, heads, kv_heads, head_dim, page_size, v_dim=None):
     assert q.dtype == out.dtype == k_cache.dtype == v_cache.dtype == torch.bfloat16
     assert block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.is_contiguous()
     assert block_table.shape[0] >= num_reqs and seq_lens.dtype == torch.int32 and seq_lens.numel() >= num_reqs
-    _check_pages(k_cache, v_cache, kv_heads, head_dim, page_size)
-    assert q.shape[1] >= heads * head_dim and out.shape[1] >= heads * head_dim
+    _check_pages(k_cache, v_cache, kv_heads, head_dim, page_size, v_dim)
+    assert q.shape[1] >= heads * head_dim and out.shape[1] >= heads * (v_dim or head_dim)
 
 
 def attn_flash(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, num_reqs: int, tokens: int,
@@ -949,17 +1098,21 @@ def attn_flash(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, num_
 def attn_flash_ext(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, num_reqs: int, max_q_len: int, *,
                    scale: float, window: int, heads: int, kv_heads: int, head_dim: int, page_size: int,
                    keep_first: int = 0, sinks: torch.Tensor | None = None, slope_exp: float = 0.0,
-                   out_scale: float = 1.0) -> torch.Tensor:
-    """The matrix-core flash kernel with the options of attn_paged_ext (bfloat16, values of the keys' size, in value
-    pages), for prompt portions and single rows alike."""
-    _need_gpu(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, sinks)
-    _check_paged(q, out, k_cache, v_cache, block_table, seq_lens, num_reqs, heads, kv_heads, head_dim, page_size)
+                   out_scale: float = 1.0, v_dim: int | None = None,
+                   sigmoid_bias: torch.Tensor | None = None) -> torch.Tensor:
+    """The matrix-core flash kernel with the options of attn_paged_ext (bfloat16, sizes attn_flash_ext_supports names,
+    values in value pages), for prompt portions and single rows alike."""
+    _need_gpu(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, sinks, sigmoid_bias)
+    vd = head_dim if v_dim is None else v_dim
+    _check_paged(q, out, k_cache, v_cache, block_table, seq_lens, num_reqs, heads, kv_heads, head_dim, page_size, vd)
+    if sigmoid_bias is not None:
+        assert sinks is None and sigmoid_bias.dtype == torch.float32 and sigmoid_bias.numel() == heads
     if sinks is not None:
         assert sinks.dtype == torch.float32 and sinks.numel() == heads and sinks.is_contiguous()
     lib.call("dinfer_attn_flash_ext", q.data_ptr(), _rows(q), out.data_ptr(), _rows(out), k_cache.data_ptr(),
              v_cache.data_ptr(), block_table.data_ptr(), block_table.shape[1], cu_seqlens.data_ptr(), seq_lens.data_ptr(),
              num_reqs, max_q_len, float(scale), int(window), int(keep_first), _ptr(sinks), float(slope_exp),
-             float(out_scale), heads, kv_heads, head_dim, page_size, _stream())
+             float(out_scale), heads, kv_heads, head_dim, vd, page_size, _ptr(sigmoid_bias), _stream())
     return out
 
 

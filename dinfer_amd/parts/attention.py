@@ -15,7 +15,12 @@ root mean square a head without a gain (`qk_unit_eps`); a query that grows with 
 (`sink_value`: 0.0 adds one to the softmax's denominator); the concatenated heads multiplied by an activation of one
 more projection of the mixer's input before the output projection (`gate`: "sigmoid" or "silu"; with `gate_heads` the
 projection gives one number a head, which multiplies all of the head's values); a learned temperature a head that
-multiplies the head's scores (`head_temp`, a tensor [heads]; it rides on the query, in the per-head norm). A layer that uses any
+multiplies the head's scores (`head_temp`, a tensor [heads]; it rides on the query, in the per-head norm); norms of q and
+of k over the whole projection, all heads of a token sharing one root mean square (`qk_row_eps`, gains of the projection's
+size); weights that are sigmoids of the scores plus a learned bias a head, not normalised over the keys (`sigmoid_bias`, a
+tensor [heads]); a bias on the output projection (`out_bias`); values mixed with another layer's (`value_mix`, a tensor of
+one number, lambda): the layer with "keep" leaves its values of the step where they are until the step's end, a layer with
+"mix" caches (1 - lambda) v + lambda v_kept of the same token. A layer that uses any
 option runs the flash kernel with options on the matrix cores where its sizes allow, else the plain kernel with options
 (csrc/attention_ref.hip), for prompt portions and single rows alike; the matrix-core kernels serve the others.
 """
@@ -39,14 +44,17 @@ class Attention(Mixer):
 
     NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight",
              "q_norm": "q_norm.", "k_norm": "k_norm.", "sink": "sinks", "q_bias": "q_proj.bias", "k_bias": "k_proj.bias",
-             "v_bias": "v_proj.bias", "g": "g_proj.weight", "temp": "temp"}
+             "v_bias": "v_proj.bias", "g": "g_proj.weight", "temp": "temp", "sigmoid_bias": "sigmoid_bias",
+             "o_bias": "o_proj.bias", "value_mix": "value_mix"}
 
     def __init__(self, hidden: int, heads: int, kv_heads: int, head_dim: int, position: PartSpec,
                  qk_norm: PartSpec | None = None, window: int | None = None, scale: float | None = None,
                  v_dim: int | None = None, keep_first: int = 0, sink: bool = False, slope_exp: float = 0.0,
                  values_are_keys: bool = False, out_scale: float = 1.0, names: dict | None = None, bias: bool = False,
                  qk_unit_eps: float | None = None, q_temp: tuple | None = None, sink_value: float | None = None,
-                 gate: str | None = None, gate_heads: bool = False, head_temp: bool = False):
+                 gate: str | None = None, gate_heads: bool = False, head_temp: bool = False,
+                 qk_row_eps: float | None = None, sigmoid_bias: bool = False, out_bias: bool = False,
+                 value_mix: str | None = None):
         if heads % kv_heads:
             raise ValueError(f"heads {heads} not divisible by kv_heads {kv_heads}")
         if head_dim <= 0 or head_dim > ops.MAX_HEAD_DIM:   # said at build, not at the first step
@@ -80,22 +88,34 @@ class Attention(Mixer):
             raise ValueError("attention: a temperature a head needs a per-head norm of q (it rides in it)")
         if self.bias and self.values_are_keys:
             raise ValueError("attention: biases with values that are the keys are not built")
+        self.qk_row_eps = None if qk_row_eps is None else float(qk_row_eps)
+        self.sigmoid, self.out_bias_on, self.value_mix = bool(sigmoid_bias), bool(out_bias), value_mix
+        if self.qk_row_eps is not None and (qk_norm is not None or qk_unit_eps is not None or self.values_are_keys):
+            raise ValueError("attention: norms over the whole projection beside per-head norms, or with values that are the "
+                             "keys, are not built")
+        if self.sigmoid and (self.sink or self.sink_value is not None):
+            raise ValueError("attention: sigmoid weights have no denominator for a sink")
+        if value_mix not in (None, "keep", "mix") or (value_mix and (self.bias or self.values_are_keys)):
+            raise ValueError(f"attention: value_mix {value_mix!r} (known: 'keep', 'mix'; without biases and with values of "
+                             "their own)")
         # what the matrix-core kernels do not do runs through the plain kernel with options
         self.extended = bool(self.v_dim != head_dim or self.keep_first or self.sink or self.slope_exp
                              or self.values_are_keys or self.out_scale != 1.0 or self.bias or qk_unit_eps is not None
                              or self.q_temp is not None or self.sink_value is not None or gate is not None
-                             or self.head_temp)
+                             or self.head_temp or self.qk_row_eps is not None or self.sigmoid or self.out_bias_on
+                             or value_mix is not None)
         self.q_size, self.kv_size = heads * head_dim, kv_heads * head_dim
         self.v_size = 0 if self.values_are_keys else kv_heads * self.v_dim
         self.g_size = (heads if self.gate_heads else heads * self.v_dim) if gate is not None else 0
         self.temps = None
         self.g_off = self.q_size + self.kv_size + self.v_size
         self.qkv = Linear(hidden, self.q_size + self.kv_size + self.v_size + self.g_size)
-        self.bias_vec = self.unit_gain = None
+        self.bias_vec = self.unit_gain = self.row_gains = self.sigmoid_biases = self.o_bias = self.kept_values = None
+        self.value_share = 0.0
         self.o = Linear(heads * self.v_dim, hidden)
         self.sinks = None
-        # decided in bind: the matrix-core flash kernel with options serves bfloat16 layers whose values have the keys'
-        # size; it reads values from transposed pages, so a layer whose values are its keys keeps them there as well
+        # decided in bind: the matrix-core flash kernel with options serves the bfloat16 layers whose sizes it takes; it
+        # reads values from transposed pages, so a layer whose values are its keys keeps them there as well
         self.mfma_ext = False
         self.stores_values = not self.values_are_keys
         self.position = POSITION_ENCODINGS.get(position.kind)(head_dim=head_dim, **position.params)
@@ -132,6 +152,15 @@ class Attention(Mixer):
             t[nm["g"]] = TensorSpec((self.g_size, Hd))
         if self.head_temp:
             t[nm["temp"]] = TensorSpec((self.heads,), init="gain")
+        if self.qk_row_eps is not None:
+            t[nm["q_norm"]] = TensorSpec((self.q_size,), init="gain")
+            t[nm["k_norm"]] = TensorSpec((self.kv_size,), init="gain")
+        if self.sigmoid:
+            t[nm["sigmoid_bias"]] = TensorSpec((self.heads,), init="zeros")
+        if self.out_bias_on:
+            t[nm["o_bias"]] = TensorSpec((Hd,), init="zeros")
+        if self.value_mix is not None:
+            t[nm["value_mix"]] = TensorSpec((), init="shares")
         for n, spec in self.position.tensors().items():   # an encoding with parameters of its own (rotations have none)
             t["position." + n] = spec
         return t
@@ -158,9 +187,14 @@ class Attention(Mixer):
     def out_weight(self, get) -> torch.Tensor:
         return get(self.names["o"], compute=True)
 
+    def out_bias(self, get) -> torch.Tensor | None:
+        """What the output projection adds (float32), for whoever runs that projection."""
+        return get(self.names["o_bias"]).float().contiguous() if self.out_bias_on else None
+
     def load(self, get):
         self.qkv.set_weight(self.weight_rows(get))
         self.o.set_weight(self.out_weight(get))
+        self.o_bias = self.out_bias(get)
         self.load_small(get)
 
     def load_small(self, get):
@@ -177,6 +211,12 @@ class Attention(Mixer):
             self.bias_vec = torch.cat([get(nm[k]).float() for k in ("q_bias", "k_bias", "v_bias")]).contiguous()
         if self.head_temp:
             self.temps = get(nm["temp"]).float().contiguous()
+        if self.qk_row_eps is not None:
+            self.row_gains = tuple(get(nm[k]).float().contiguous() for k in ("q_norm", "k_norm"))
+        if self.sigmoid:
+            self.sigmoid_biases = get(nm["sigmoid_bias"]).float().contiguous()
+        if self.value_mix == "mix":      # (the layer that keeps its values has the tensor too and does not use it)
+            self.value_share = float(get(nm["value_mix"]).float())
         if self.qk_unit_eps is not None:
             self.unit_gain = torch.ones(self.head_dim, dtype=torch.float32, device=some.device)
         self.position.load(lambda n, **kw: get("position." + n, **kw))
@@ -184,14 +224,22 @@ class Attention(Mixer):
     def bind_core(self, ctx):
         self.page_size = ctx.page_size
         self.position.bind(ctx)
-        self.mfma_ext = bool(ctx.dtype == torch.bfloat16 and self.v_dim == self.head_dim
-                             and ops.attn_mfma_supports(self.head_dim, ctx.page_size, self.heads, self.kv_heads))
+        self.mfma_ext = bool(ctx.dtype == torch.bfloat16
+                             and ops.attn_flash_ext_supports(self.head_dim, self.v_dim, ctx.page_size, self.heads,
+                                                             self.kv_heads, self.sigmoid))
         self.stores_values = not self.values_are_keys or self.mfma_ext
 
     def bind(self, ctx):
         ws = ctx.workspace
         self.bind_core(ctx)
-        self.qkv_buf = ws.buffer("qkv", self.qkv.out_features)
+        # (a layer whose values later layers read has a buffer no other layer writes)
+        self.qkv_buf = ws.buffer("qkv" if self.value_mix != "keep" else "qkv_kept", self.qkv.out_features)
+        if self.value_mix is not None:
+            v_off = self.q_size + self.kv_size
+            kept = ctx.share("kept_values", lambda: self.qkv_buf[:, v_off:v_off + self.v_size] if self.value_mix == "keep" else None)
+            if kept is None or kept.shape[1] != self.v_size or (self.value_mix == "keep") != (kept.data_ptr() == self.qkv_buf[:, v_off:].data_ptr()):
+                raise ValueError("attention: values are mixed with those of one earlier layer that keeps values of the same size")
+            self.kept_values = kept if self.value_mix == "mix" else None
         self.attn_buf = ws.buffer("attn", self.heads * self.v_dim)
         self.out_buf = ws.buffer("mixer_out", self.hidden)
         self.attn_ws = attn_kernels.Workspace(ctx, self.heads, self.kv_heads, self.head_dim)
@@ -208,6 +256,8 @@ class Attention(Mixer):
         outputs go to column `out_col` of attn_buf (a mixer that joins several shares one product on each side)."""
         T = batch.num_tokens
         g = cache.group
+        if self.value_mix is not None and qkv_buf is not self.qkv_buf:
+            raise NotImplementedError("attention: values are not mixed inside a joined mixer")
         if self.extended or col or out_col:
             return self._core_ext(qkv_buf, col, attn_buf, out_col, batch, cache)
         qn, pos = self.q_norm, self.position
@@ -256,6 +306,8 @@ class Attention(Mixer):
         vd = self.v_dim
         q_gain, k_gain = (qn.weight, self.k_norm.weight) if qn else (self.unit_gain, self.unit_gain)
         eps = qn.eps if qn else (self.qk_unit_eps or 0.0)
+        if self.row_gains is not None:
+            (q_gain, k_gain), eps = self.row_gains, self.qk_row_eps
         ops.qkv_post(qkv_buf, T, heads=self.heads, kv_heads=self.kv_heads, head_dim=self.head_dim, q_off=col,
                      k_off=col + self.q_size,     # (values that are the keys: the key columns as the product left them)
                      v_off=col + self.q_size + (0 if self.values_are_keys else self.kv_size),
@@ -263,7 +315,9 @@ class Attention(Mixer):
                      q_gain=q_gain, k_gain=k_gain, eps=eps, gain_offset=qn.weight_offset if qn else 0.0,
                      cos_sin=pos.table(), rotary_dim=pos.rotary_dim, rope_style=pos.style,
                      k_cache=cache.k, v_cache=cache.v, slot_mapping=batch.slot_mapping[g] if cache.owner else None,
-                     token_runs=False, v_dim=vd, bias=self.bias_vec, q_temp=self.q_temp, q_head_scale=self.temps)
+                     token_runs=batch.max_q_len >= 8, v_dim=vd, bias=self.bias_vec, q_temp=self.q_temp,
+                     q_head_scale=self.temps, whole=self.row_gains is not None, v_first=self.kept_values,
+                     v_share=self.value_share)
         self._attend_ext(qkv_buf, col, attn_buf, out_col, batch, cache)
         if self.gate is not None:
             n = self.heads * vd
@@ -277,17 +331,21 @@ class Attention(Mixer):
                                batch.cu_seqlens, batch.seq_lens, batch.num_reqs, batch.max_q_len, scale=self.scale,
                                window=self.window or 0, heads=self.heads, kv_heads=self.kv_heads, head_dim=self.head_dim,
                                page_size=self.page_size, keep_first=self.keep_first, sinks=self.sinks,
-                               slope_exp=self.slope_exp, out_scale=self.out_scale)
+                               slope_exp=self.slope_exp, out_scale=self.out_scale, v_dim=vd,
+                               sigmoid_bias=self.sigmoid_biases)
             return
         ops.attn_paged_ext(qkv_buf[:, col:], attn_buf[:, out_col:], cache.k, cache.v, batch.block_table[g],
                            batch.cu_seqlens, batch.seq_lens, batch.num_reqs, T, scale=self.scale,
                            window=self.window or 0, heads=self.heads, kv_heads=self.kv_heads, head_dim=self.head_dim,
                            page_size=self.page_size, v_dim=vd, keep_first=self.keep_first, sinks=self.sinks,
-                           slope_exp=self.slope_exp, out_scale=self.out_scale)
+                           slope_exp=self.slope_exp, out_scale=self.out_scale, sigmoid_bias=self.sigmoid_biases)
 
     def _project_out(self, T, into):
-        if into is not None:
+        if into is not None and self.o_bias is None:
             done = self.o.forward_into(self.attn_buf, into, T)
             if done is not None:
                 return done
-        return self.o.forward(self.attn_buf, self.out_buf, T, scratch=True)
+        y = self.o.forward(self.attn_buf, self.out_buf, T, scratch=True)
+        if self.o_bias is not None:
+            ops.add_rows(y, T, vec=self.o_bias)
+        return y

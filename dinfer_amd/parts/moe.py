@@ -6,7 +6,8 @@
         + sigmoid(wsg . x) * shared(x)          (a gated feed-forward every token runs, where the layer has one)
 
 (The softmax over the chosen logits is the softmax over all experts with the chosen scores divided by their sum.)
-With `gated=False` an expert, and the shared one, is down_e( act(up_e x) ) with act "silu" or "gelu" (error function);
+With `gated=False` an expert, and the shared one, is down_e( act(up_e x) ) with act "silu", "gelu" (error function) or
+"relu2" (the square of relu);
 with `shared_gate=False` the shared expert's output is added as it is.
 
 Another rule of routing (`scores="all"`): the scores are the softmax of z over all router outputs; the `top` largest
@@ -14,6 +15,11 @@ of score + correction are chosen (`correction`, a tensor of one number a router 
 chosen expert's weight is its score as it is, so a token's weights need not sum to one. `identity` experts: the router
 has `experts + identity` outputs, and the last `identity` of them stand for experts without tensors whose output is
 their input (times the weight).
+
+A third (`scores="sigmoid"`): the scores are the sigmoids of the logits, each by itself; the `top` largest are chosen and
+weigh as they are. `weigh="input"`: a chosen expert's weight multiplies what goes into the expert instead of what comes
+out, y = sum_chosen expert_e(p_e x); the first product is linear in its input, so the weight multiplies its float sums
+before the activation. With one choice a token its expert's row is the layer's output, and nothing is left to sum.
 
 Per step: one kernel routes (logits, choice, weights, the shared gate), one sorts the (token, choice) entries by
 expert and writes the work list of row tiles, two launches run the products of all experts (gate and up with the
@@ -40,15 +46,20 @@ class RoutedExperts(FeedForward):
 
     def __init__(self, hidden: int, experts: int, top: int, intermediate: int, shared_intermediate: int | None = None,
                  act: str = "silu", gated: bool = True, shared_gate: bool = True, scores: str = "chosen",
-                 correction: bool = False, identity: int = 0):
+                 correction: bool = False, identity: int = 0, weigh: str = "output"):
         if gated and act != "silu":
             raise ValueError(f"routed feed-forward: gated activation {act!r} has no kernel (known: ['silu'])")
         if not gated and act not in ops.EXPERT_ACTS:
             raise ValueError(f"routed feed-forward: activation {act!r} has no kernel (known: {sorted(ops.EXPERT_ACTS)})")
-        if scores not in ("chosen", "all") or identity < 0 or (scores != "all" and (correction or identity)):
+        if weigh not in ("output", "input") or (weigh == "input" and (identity or shared_intermediate)):
+            raise ValueError(f"routed feed-forward: weights on the {weigh!r} with {identity} identity experts or a shared one "
+                             "are not built (known: 'output', and 'input' for routed experts alone)")
+        self.weigh_input = weigh == "input"
+        if scores not in ("chosen", "all", "sigmoid") or identity < 0 or (scores != "all" and (correction or identity)):
             raise ValueError(f"routed feed-forward: scores {scores!r} with correction {correction} and {identity} identity "
                              "experts: a correction and identity experts go with scores over all router outputs")
-        self.all_scores, self.has_correction, self.identity = scores == "all", bool(correction), int(identity)
+        self.all_scores = {"chosen": 0, "all": 1, "sigmoid": 2}[scores]
+        self.has_correction, self.identity = bool(correction), int(identity)
         self.outputs = experts + self.identity          # what the router gives a token
         if not (0 < top <= self.outputs) or self.outputs > ops.MOE_MAX_EXPERTS or top > ops.MOE_MAX_TOP:
             raise ValueError(f"routed feed-forward: {top} of {experts} experts has no kernel (up to {ops.MOE_MAX_TOP} of "
@@ -121,10 +132,14 @@ class RoutedExperts(FeedForward):
         rows = ops.moe_tile_rows(self.dtype, n, self.outputs, self.hidden, self.intermediate)   # follows the step's count alone
         ops.moe_scatter(self.idx, n, self.outputs, self.offsets, self.perm, self.tiles, rows, real_experts=self.experts)
         ops.experts_nt(x, self.w_in, self.act_buf, n, self.tiles, self.offsets, self.perm, gated=self.gated, a_div=top,
-                       c_to_perm=False, tile_rows=rows, act=None if self.gated else self.act)
-        ops.experts_nt(self.act_buf, self.w_out, self.y_buf, n, self.tiles, self.offsets, self.perm, gated=False, a_div=0,
+                       c_to_perm=False, tile_rows=rows, act=None if self.gated else self.act,
+                       row_scale=self.share if self.weigh_input else None)
+        alone = self.weigh_input and top == 1      # a token's one row of the second product is its output
+        ops.experts_nt(self.act_buf, self.w_out, self.out_buf if alone else self.y_buf, n, self.tiles, self.offsets, self.perm, gated=False, a_div=0,
                        c_to_perm=True, tile_rows=rows)
+        if alone:
+            return self.out_buf
         shared = self.shared.forward(x, batch) if self.shared is not None else None
         same = dict(idx=self.idx, real_experts=self.experts, x=x) if self.identity else {}
-        return ops.moe_combine(self.y_buf, self.share, top, shared, self.shared_gate if self.sg is not None else None,
+        return ops.moe_combine(self.y_buf, None if self.weigh_input else self.share, top, shared, self.shared_gate if self.sg is not None else None,
                                self.out_buf, T, **same)

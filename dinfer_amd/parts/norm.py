@@ -1,7 +1,9 @@
 """RMSNorm: y = x / sqrt(mean(x^2) + eps) * (w + offset), float arithmetic
 (crates/layers/src/nn.rs:78-111, crates/kernels/cuda/rmsnorm_core.cuh:63-81).
 LayerNorm: y = (x - mean) / sqrt(var + eps) * w + b, float arithmetic; its input (the residual stream) may be kept in
-32 bits where its output is the engine's dtype."""
+32 bits where its output is the engine's dtype.
+Group RMSNorm: the row in equal consecutive parts, each divided by its own root mean square, times a gain an entry; it
+reads a stream in any storage type."""
 from __future__ import annotations
 
 from ..kernels import ops
@@ -32,6 +34,26 @@ class RMSNorm(Norm):
                                       rows=rows)
         return ops.rmsnorm(x, self.weight, out, self.eps, n_rows, residual=residual, rows=rows,
                            weight_offset=self.weight_offset)
+
+
+@NORMS.register("group_rmsnorm")
+class GroupRMSNorm(Norm):
+    """y = x_part / sqrt(mean(x_part^2) + eps) * w, `groups` equal consecutive parts a row (one: a plain RMSNorm)."""
+
+    def __init__(self, width: int, eps: float, groups: int = 1, weight_name: str = "weight"):
+        if groups <= 0 or width % groups:
+            raise ValueError(f"group norm: {groups} groups do not divide a width of {width}")
+        self.width, self.eps, self.groups, self.weight_name = width, float(eps), int(groups), weight_name
+        self.weight = None
+
+    def tensors(self):
+        return {self.weight_name: TensorSpec((self.width,), init="gain")}
+
+    def load(self, get):
+        self.weight = get(self.weight_name).float().contiguous()      # (exact for a bfloat16 file)
+
+    def forward(self, x, out, n_rows, *, residual=None, rows=None):
+        return ops.group_rmsnorm(x, self.weight, out, self.eps, n_rows, self.groups, residual=residual, rows=rows)
 
 
 @NORMS.register("layernorm")
