@@ -8,6 +8,7 @@
     python bench.py --workload karopel [--karopel-shape 2k|4k] [--layers 4] [--prompt 2048] [--only karopel|qwen3]
     python bench.py --workload fanulix [--fanulix-shape 2k|4k] [--layers 4] [--prompt 2048] [--only fanulix|karopel|qwen3]
     python bench.py --workload verorax [--verorax-shape 2k|4k] [--layers 4] [--prompt 2048] [--only verorax|kudurax|karopel|qwen3]
+    python bench.py --workload lotelix [--lotelix-shape 2k|4k] [--layers 4] [--prompt 2048] [--only lotelix|fanulix|karopel|qwen3]
 
 Prints ONE JSON line. `value` is decoded tokens per second at the default batch (8), each
 request with a 2,048-token prompt in a 4,096-token context; a "step" is one decode step
@@ -345,6 +346,50 @@ def verorax(a, torch, Engine, SamplingParams) -> int:
                         VeroraxConfig.from_dict(verorax_config(shape, layers, 32768)), beside=beside)
 
 
+# Lotelix layer sizes that resemble a real model's: an attention with sigmoid weights and grouped keys and values beside a
+# gated linear attention of as many heads, all heads 128 wide, a decay projection of 16 inside; a minGRU of the model's
+# width; an attention with a window of 1,024, sinks and mixed values; 64 routed experts of which a token uses 6. Beside
+# them Fanulix layers of the same width (the closest design: an attention with options beside a linear recurrence, routed
+# experts without gates), Karopel and Qwen3 layers
+LOTELIX_SHAPES = {
+    "2k": dict(width=2048, heads=16, kv_heads=4, dim=128, window=1024, gla_heads=16, decay_rank=16, gru=2048, groups=4,
+               experts=64, top=6, expert_ff=1408, fanulix="2k", karopel="2k",
+               qwen=dict(num_attention_heads=16, num_key_value_heads=4, head_dim=128, intermediate_size=8192)),
+    "4k": dict(width=4096, heads=32, kv_heads=8, dim=128, window=1024, gla_heads=32, decay_rank=16, gru=4096, groups=8,
+               experts=64, top=8, expert_ff=1536, fanulix="4k", karopel="4k",
+               qwen=dict(num_attention_heads=32, num_key_value_heads=8, head_dim=128, intermediate_size=12288)),
+}
+
+
+def lotelix_config(shape: dict, layers: int, vocab: int) -> dict:
+    """Layers in fours: parallel, minGRU, attention, attention; every layer with routed experts."""
+    d = shape["dim"]
+    moe = dict(kind="moe", expert=dict(ff=shape["expert_ff"]), router=dict(experts=shape["experts"], top=shape["top"]))
+    heads = dict(heads=shape["heads"], kv_heads=shape["kv_heads"], dim=d, vdim=d, scale=d ** -0.5)
+    par = dict(left=dict(heads, rot=dict(base=1000000.0, dims=d)),
+               right=dict(heads=shape["gla_heads"], dim=d, vdim=d, tau=16.0, decay_rank=shape["decay_rank"]))
+    att = dict(heads, mask=dict(size=shape["window"]), v_mix=True,
+               rot=dict(base=500000.0, dims=d, scaling=dict(factor=8.0, low=1.0, high=4.0, original=8192)))
+    four = [dict(type="parallel", mixer=par, mlp=moe), dict(type="mingru", mixer=dict(width=shape["gru"]), mlp=moe),
+            dict(type="attention", mixer=att, mlp=moe), dict(type="attention", mixer=att, mlp=moe)]
+    return dict(architecture="Lotelix", vocab=vocab, width=shape["width"], embedding=dict(scale=1.0),
+                norm=dict(eps=1e-5, groups=shape["groups"]), layers=[four[i % 4] for i in range(layers)])
+
+
+def lotelix(a, torch, Engine, SamplingParams) -> int:
+    """Prefill and decode throughput of Lotelix layers of a real model's sizes beside Fanulix, Karopel and Qwen3 layers of
+    the same width."""
+    from dinfer_amd.config.fanulix import FanulixConfig
+    from dinfer_amd.config.karopel import KaropelConfig
+    from dinfer_amd.config.lotelix import LotelixConfig
+    shape = LOTELIX_SHAPES[a.lotelix_shape]
+    layers = a.layers or 4
+    beside = {"fanulix": FanulixConfig.from_dict(fanulix_config(FANULIX_SHAPES[shape["fanulix"]], layers, 32768)),
+              "karopel": KaropelConfig.from_dict(karopel_config(KAROPEL_SHAPES[shape["karopel"]], layers, 32768))}
+    return beside_qwen3(a, torch, Engine, SamplingParams, "lotelix", "Lotelix", a.lotelix_shape, shape,
+                        LotelixConfig.from_dict(lotelix_config(shape, layers, 32768)), beside=beside)
+
+
 def fanulix(a, torch, Engine, SamplingParams) -> int:
     """Prefill and decode throughput of Fanulix layers of a real model's sizes beside Karopel and Qwen3 layers of the same
     width."""
@@ -465,9 +510,11 @@ def main() -> int:
     ap.add_argument("--karopel-shape", default="2k", choices=sorted(KAROPEL_SHAPES), help="karopel: layer sizes")
     ap.add_argument("--fanulix-shape", default="2k", choices=sorted(FANULIX_SHAPES), help="fanulix: layer sizes")
     ap.add_argument("--verorax-shape", default="2k", choices=sorted(VERORAX_SHAPES), help="verorax: layer sizes")
-    ap.add_argument("--only", default="", choices=["", "kudurax", "karopel", "fanulix", "verorax", "qwen3"],
-                    help="kudurax, karopel, fanulix: measure one of the models")
-    ap.add_argument("--workload", default="decode", choices=["decode", "serving", "closed", "kudurax", "karopel", "fanulix", "verorax"],
+    ap.add_argument("--lotelix-shape", default="2k", choices=sorted(LOTELIX_SHAPES), help="lotelix: layer sizes")
+    ap.add_argument("--only", default="", choices=["", "kudurax", "karopel", "fanulix", "verorax", "lotelix", "qwen3"],
+                    help="kudurax, karopel, fanulix, verorax, lotelix: measure one of the models")
+    ap.add_argument("--workload", default="decode", choices=["decode", "serving", "closed", "kudurax", "karopel", "fanulix", "verorax",
+                                                                  "lotelix"],
                     help="serving: 32 requests with prompts of 512 to 3,072 tokens fed in portions of 512 beside the "
                          "requests that decode, 256 outputs each (meant for the 14B shape); closed: --concurrency "
                          "requests live at any time, --prompt tokens in and --max-tokens out each, the load of the "
@@ -495,6 +542,8 @@ def main() -> int:
         return karopel(a, torch, Engine, SamplingParams)
     if a.workload == "verorax":
         return verorax(a, torch, Engine, SamplingParams)
+    if a.workload == "lotelix":
+        return lotelix(a, torch, Engine, SamplingParams)
     if a.workload == "fanulix":
         return fanulix(a, torch, Engine, SamplingParams)
     if a.workload == "serving":

@@ -26,6 +26,7 @@ constexpr int CH = 16;          // tokens whose operands wait in LDS
 constexpr int CL = 128;         // tokens of a chunk (a multiple of CH)
 constexpr int LOW_TOKENS = 8;
 constexpr int MAX_LOW = 512;
+constexpr float LOG2E = 1.4426950408889634f;
 
 template <class S, int TT>
 __global__ void __launch_bounds__(256) channel_decay_kernel(const S* __restrict__ proj, int64_t ld, int64_t low_off, int low,
@@ -53,8 +54,11 @@ __global__ void __launch_bounds__(256) channel_decay_kernel(const S* __restrict_
   }
 #pragma unroll
   for (int t = 0; t < TT; ++t) {
-    const float log_sigmoid = fminf(z[t], 0.f) - log1pf(expf(-fabsf(z[t])));
-    if (t < nt) out[(int64_t)(t0 + t) * ld_out + c] = expf(log_sigmoid * inv_tau);
+    // log2 sigmoid(z) = min(y, 0) - log2(1 + 2^-|y|), y = z log2(e); the logarithm of one and next to nothing as the
+    // first terms of its series, or the slow decays would lose what sets them apart from one
+    const float y = z[t] * LOG2E, e = __builtin_amdgcn_exp2f(-fabsf(y));
+    const float l = e < 0.0078125f ? LOG2E * e * (1.f - e * (0.5f - e * (1.f / 3.f))) : __builtin_amdgcn_logf(1.f + e);
+    if (t < nt) out[(int64_t)(t0 + t) * ld_out + c] = __builtin_amdgcn_exp2f((fminf(y, 0.f) - l) * inv_tau);
   }
 }
 

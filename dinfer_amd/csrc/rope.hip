@@ -459,26 +459,18 @@ __global__ void __launch_bounds__(WAVES * 64) qkv_post_vec_kernel(
 }
 
 // Norms over the whole projection: all q heads of a token share one root mean square, all k heads another (gains
-// [H D] and [Hkv D], float), before the rotation. A workgroup takes a token: the row waits in LDS as floats between the
-// sums and the rotation, which reads a pair's other element there. P: entries a thread takes at a time (8: bf16 rows of
-// whole 16-byte pieces that no boundary of a head, of its rotated part or of that part's halves cuts; else 1).
-// gather_v as in qkv_post_vec_kernel (P = 8 only).
-template <class S, int P>
+// [H D] and [Hkv D], float), before the rotation.
+//
+// Any sizes and types: a workgroup takes a token, the row waits in LDS as floats between the sums and the rotation, which
+// reads a pair's other element there.
+template <class S>
 __global__ void __launch_bounds__(256) qkv_row_post_kernel(
     S* __restrict__ qkv, int64_t ld, int64_t q_off, int64_t k_off, int64_t v_off, const float* __restrict__ wq,
     const float* __restrict__ wk, float eps, const int32_t* __restrict__ pos, const float* __restrict__ cos_sin, int rot,
     int style, S* __restrict__ k_cache, S* __restrict__ v_cache, const int64_t* __restrict__ slots, int H, int Hkv, int D,
-    int page, int Dv, const float* __restrict__ bias, int tokens, int gather_v, ValueMix mix) {
+    int page, int Dv, const float* __restrict__ bias, ValueMix mix) {
   extern __shared__ __attribute__((aligned(16))) float row_smem[];
   __shared__ float red[16];
-  if constexpr (P == 8) {
-    if ((int)blockIdx.x >= tokens) {
-      const int j = (int)blockIdx.x - tokens;
-      v_write_transposed((const bf16*)qkv, ld, v_off, (bf16*)v_cache, slots, tokens, Hkv, Dv, page, j / Hkv, j % Hkv,
-                         bias ? bias + (int64_t)(H + Hkv) * D + (int64_t)(j % Hkv) * Dv : nullptr, mix);
-      return;
-    }
-  }
   const int64_t t = blockIdx.x;
   S* row = qkv + t * ld;
   const int64_t slot = slots ? slots[t] : -1;
@@ -486,70 +478,189 @@ __global__ void __launch_bounds__(256) qkv_row_post_kernel(
   const int off = slot >= 0 ? (int)(slot % page) : 0;
   const int nq = H * D, n = nq + Hkv * D;
   float sq = 0.f, sk = 0.f;
-  for (int i = threadIdx.x * P; i < n; i += 256 * P) {
-    const S* src = i < nq ? row + q_off + i : row + k_off + (i - nq);
-    float v[P];
-    if constexpr (P == 8) {
-      const bf16x8 x = *(const bf16x8*)src;
-#pragma unroll
-      for (int e = 0; e < P; ++e) v[e] = (float)x[e];
-    } else {
-      v[0] = to_f32(src[0]);
-    }
-#pragma unroll
-    for (int e = 0; e < P; ++e) {
-      if (bias) v[e] += bias[i + e];
-      row_smem[i + e] = v[e];
-      if (i < nq) sq = add_square(sq, v[e]);
-      else sk = add_square(sk, v[e]);
-    }
+  for (int i = threadIdx.x; i < n; i += 256) {
+    float v = to_f32(i < nq ? row[q_off + i] : row[k_off + (i - nq)]);
+    if (bias) v += bias[i];
+    row_smem[i] = v;
+    if (i < nq) sq = add_square(sq, v);
+    else sk = add_square(sk, v);
   }
   // (the barriers inside also publish the row)
   const float fq = 1.f / sqrtf(block_sum(sq, red) / (float)nq + eps);
   const float fk = 1.f / sqrtf(block_sum(sk, red) / (float)(n - nq) + eps);
   const float* cs = cos_sin ? cos_sin + (int64_t)pos[t] * rot : nullptr;
   const int half = rot / 2, Dp = (D + 7) & ~7;
-  for (int i = threadIdx.x * P; i < n; i += 256 * P) {
+  for (int i = threadIdx.x; i < n; i += 256) {
     const bool is_q = i < nq;
     const int e0 = is_q ? i : i - nq, hd = e0 / D, d = e0 - hd * D;
     const float* w = is_q ? wq : wk;
     const float f = is_q ? fq : fk;
-    float y[P];
-#pragma unroll
-    for (int e = 0; e < P; ++e) y[e] = row_smem[i + e] * f * w[e0 + e];
+    float y = row_smem[i] * f * w[e0];
     if (cs && d < rot) {
-      float r[P];
-#pragma unroll
-      for (int e = 0; e < P; ++e) {
-        const int de = d + e;
-        const bool first = style == 0 ? de < half : (de & 1) == 0;
-        const int pi = style == 0 ? (first ? de : de - half) : de >> 1;
-        const int step = style == 0 ? half : 1, other = first ? step : -step;
-        const float o = row_smem[i + e + other] * f * w[e0 + e + other];
-        r[e] = first ? rotated_first(y[e], o, cs[pi], cs[half + pi]) : rotated_second(o, y[e], cs[pi], cs[half + pi]);
-      }
-#pragma unroll
-      for (int e = 0; e < P; ++e) y[e] = r[e];
+      const bool first = style == 0 ? d < half : (d & 1) == 0;
+      const int pi = style == 0 ? (first ? d : d - half) : d >> 1;
+      const int step = style == 0 ? half : 1, other = first ? step : -step;
+      const float o = row_smem[i + other] * f * w[e0 + other];
+      y = first ? rotated_first(y, o, cs[pi], cs[half + pi]) : rotated_second(o, y, cs[pi], cs[half + pi]);
     }
-    S* to = is_q ? row + q_off + e0
-                 : !slots ? row + k_off + e0
-                          : slot >= 0 ? k_cache + (blk * Hkv + hd) * (int64_t)page * Dp + k_page_offset(off, d, page) : nullptr;
-    if (!to) continue;
-    if constexpr (P == 8) {
-      bf16x8 r;
-#pragma unroll
-      for (int e = 0; e < P; ++e) r[e] = (bf16)y[e];
-      *(bf16x8*)to = r;
-    } else {
-      to[0] = from_f32<S>(y[0]);
-    }
+    const S r = from_f32<S>(y);
+    if (is_q) row[q_off + e0] = r;
+    else if (!slots) row[k_off + e0] = r;
+    else if (slot >= 0) k_cache[(blk * Hkv + hd) * (int64_t)page * Dp + k_page_offset(off, d, page)] = r;
   }
-  if (slot < 0 || !v_cache || gather_v > 0) return;
+  if (slot < 0 || !v_cache) return;
   for (int i = threadIdx.x; i < Hkv * Dv; i += 256) {
     float v = to_f32(row[v_off + i]);
     if (bias) v += bias[n + i];
     if (mix.first) v = mixed_value<S>(v, mix, t, i);
     v_cache[(blk * Hkv * Dv + i) * (int64_t)page + off] = from_f32<S>(v);
+  }
+}
+
+// bf16 rows of whole 16-byte pieces that no boundary of a head, of its rotated part or (style 0) of that part's halves cuts:
+// a thread owns one piece of 8 entries (ITERS of them) of q | k and keeps its bias and gains in registers for the per_block
+// tokens its workgroup goes through, one after the other with the next one's piece on its way. Pairs (2i, 2i + 1) lie in a
+// piece; for pairs (i, i + rot/2) the row passes through LDS. gather_v as in qkv_post_vec_kernel: then the workgroups from
+// blockIdx.x = `blocks` on write V (8 * WAVES tokens of a kv head each, by their first WAVES waves).
+template <int ITERS>
+__global__ void __launch_bounds__(1024) qkv_row_post_vec_kernel(
+    bf16* __restrict__ qkv, int64_t ld, int64_t q_off, int64_t k_off, int64_t v_off, const float* __restrict__ wq,
+    const float* __restrict__ wk, float eps, const int32_t* __restrict__ pos, const float* __restrict__ cos_sin, int rot,
+    int style, bf16* __restrict__ k_cache, bf16* __restrict__ v_cache, const int64_t* __restrict__ slots, int H, int Hkv,
+    int D, int page, int Dv, const float* __restrict__ bias, int tokens, int per_block, int blocks, int gather_v,
+    ValueMix mix) {
+  extern __shared__ __attribute__((aligned(16))) float row_smem[];   // style 0: the normed row
+  __shared__ float red[2][2][16];                                    // two sums a wave, two tokens in turn
+  if ((int)blockIdx.x >= blocks) {
+    const int j = (int)blockIdx.x - blocks;
+    if (threadIdx.x < WAVES * 64)
+      v_write_transposed(qkv, ld, v_off, v_cache, slots, tokens, Hkv, Dv, page, j / Hkv, j % Hkv,
+                         bias ? bias + (int64_t)(H + Hkv) * D + (int64_t)(j % Hkv) * Dv : nullptr, mix);
+    return;
+  }
+  const int nq = H * D, n = nq + Hkv * D, half = rot / 2, threads = blockDim.x;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, waves = threads >> 6;
+  int at[ITERS], d0[ITERS];
+  float g[ITERS][8], bs[ITERS][8];
+  bf16x8 x[ITERS];
+  const int first_t = blockIdx.x * per_block, last_t = first_t + per_block < tokens ? first_t + per_block : tokens;
+  auto source = [&](int t, int i) { return qkv + (int64_t)t * ld + (i < nq ? q_off + i : k_off + (i - nq)); };
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int i = 8 * (it * threads + threadIdx.x);
+    at[it] = i < n ? i : -1;
+    d0[it] = 0;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) g[it][e] = bs[it][e] = 0.f;
+    x[it] = zero8();
+    if (i >= n) continue;
+    const int e0 = i < nq ? i : i - nq;
+    d0[it] = e0 % D;
+    x[it] = *(const bf16x8*)source(first_t, i);
+    const float* w = (i < nq ? wq : wk) + e0;
+    const f32x4 a = *(const f32x4*)w, b = *(const f32x4*)(w + 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) { g[it][e] = a[e]; g[it][4 + e] = b[e]; }
+    if (bias) {
+      const f32x4 c = *(const f32x4*)(bias + i), d = *(const f32x4*)(bias + i + 4);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) { bs[it][e] = c[e]; bs[it][4 + e] = d[e]; }
+    }
+  }
+  for (int t = first_t; t < last_t; ++t) {
+    float v[ITERS][8], c[ITERS][8], sn[ITERS][8];
+    float sq = 0.f, sk = 0.f;
+    const int64_t slot = slots ? slots[t] : -1;
+    const float* cs = cos_sin ? cos_sin + (int64_t)pos[t] * rot : nullptr;
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+      if (at[it] < 0) continue;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        v[it][e] = (float)x[it][e] + bs[it][e];
+        if (at[it] < nq) sq = add_square(sq, v[it][e]);
+        else sk = add_square(sk, v[it][e]);
+      }
+      if (cs && d0[it] < rot) {      // style 1: four pairs a piece; style 0: eight, of one half
+        const int pi = style ? d0[it] / 2 : d0[it] < half ? d0[it] : d0[it] - half;
+        const f32x4 c0 = *(const f32x4*)(cs + pi), s0 = *(const f32x4*)(cs + half + pi);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) { c[it][e] = c0[e]; sn[it][e] = s0[e]; }
+        if (!style) {
+          const f32x4 c1 = *(const f32x4*)(cs + pi + 4), s1 = *(const f32x4*)(cs + half + pi + 4);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) { c[it][4 + e] = c1[e]; sn[it][4 + e] = s1[e]; }
+        }
+      }
+      if (t + 1 < last_t) x[it] = *(const bf16x8*)source(t + 1, at[it]);
+    }
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    float (&rd)[2][16] = red[(t - first_t) & 1];
+    if (lane == 0) { rd[0][wave] = sq; rd[1][wave] = sk; }
+    __syncthreads();
+    sq = sk = 0.f;
+    for (int w = 0; w < waves; ++w) { sq += rd[0][w]; sk += rd[1][w]; }      // a fixed order: the same in every thread
+    const float fq = 1.f / sqrtf(sq / (float)nq + eps), fk = 1.f / sqrtf(sk / (float)(n - nq) + eps);
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+      if (at[it] < 0) continue;
+      const float f = at[it] < nq ? fq : fk;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[it][e] = v[it][e] * f * g[it][e];
+      if (cs && !style) {
+        f32x4 a, b;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) { a[e] = v[it][e]; b[e] = v[it][4 + e]; }
+        *(f32x4*)(row_smem + at[it]) = a;
+        *(f32x4*)(row_smem + at[it] + 4) = b;
+      }
+    }
+    if (cs && !style) __syncthreads();
+    const int64_t blk = slot >= 0 ? slot / page : 0;
+    const int off = slot >= 0 ? (int)(slot % page) : 0;
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+      if (at[it] < 0) continue;
+      if (cs && d0[it] < rot) {
+        if (style) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const float u = v[it][2 * e], w = v[it][2 * e + 1];
+            v[it][2 * e] = rotated_first(u, w, c[it][e], sn[it][e]);
+            v[it][2 * e + 1] = rotated_second(u, w, c[it][e], sn[it][e]);
+          }
+        } else {
+          const bool first = d0[it] < half;
+          const float* o = row_smem + at[it] + (first ? half : -half);
+          const f32x4 o0 = *(const f32x4*)o, o1 = *(const f32x4*)(o + 4);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) {
+            const float other = e < 4 ? o0[e & 3] : o1[e & 3];
+            v[it][e] = first ? rotated_first(v[it][e], other, c[it][e], sn[it][e]) : rotated_second(other, v[it][e], c[it][e], sn[it][e]);
+          }
+        }
+      }
+      bf16x8 r;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) r[e] = (bf16)v[it][e];
+      if (at[it] < nq || !slots) {
+        *(bf16x8*)source(t, at[it]) = r;
+      } else if (slot >= 0) {
+        const int hd = (at[it] - nq) / D;
+        *(bf16x8*)(k_cache + (blk * Hkv + hd) * (int64_t)page * D + k_page_offset(off, d0[it], page)) = r;
+      }
+    }
+    if (cs && !style) __syncthreads();      // the row has been read before the next token's is written
+    if (slot >= 0 && v_cache && gather_v == 0) {
+      const bf16* vr = qkv + (int64_t)t * ld + v_off;
+      for (int i = threadIdx.x; i < Hkv * Dv; i += threads) {
+        float y = (float)vr[i];
+        if (bias) y += bias[n + i];
+        if (mix.first) y = mixed_value<bf16>(y, mix, t, i);
+        v_cache[(blk * Hkv * Dv + i) * (int64_t)page + off] = (bf16)y;
+      }
+    }
   }
 }
 
@@ -575,28 +686,38 @@ extern "C" int dinfer_qkv_row_post(int dtype, void* qkv, int64_t tokens, int64_t
   const ValueMix mix{v_first, ld_v_first, v_share};
   const int rot = cos_sin ? rotary_dim : 0;
   const bool vec = dtype == DT_BF16 && head_dim % 8 == 0 && rot % (style == 0 ? 16 : 8) == 0 && ld % 8 == 0 && q_off % 8 == 0 &&
-                   k_off % 8 == 0 && v_off % 2 == 0 && v_dim % 2 == 0 && ((uintptr_t)qkv % 16) == 0 &&
-                   ((uintptr_t)k_cache % 16) == 0;
+                   k_off % 8 == 0 && v_off % 2 == 0 && v_dim % 2 == 0 && n <= 8 * 1024 * 2 && ((uintptr_t)qkv % 16) == 0 &&
+                   ((uintptr_t)k_cache % 16) == 0 && ((uintptr_t)q_gain % 16) == 0 && ((uintptr_t)k_gain % 16) == 0 &&
+                   ((uintptr_t)bias % 16) == 0 && ((uintptr_t)cos_sin % 16) == 0;
   if (vec) {
+    const int64_t pieces = n / 8;
+    const int iters = (int)((pieces + 1023) / 1024);
+    int threads = (int)((pieces + iters - 1) / iters);
+    threads = (threads + 63) / 64 * 64;
     const bool gather = slot_mapping && v_cache && token_runs && tokens >= 64 && page_size % 8 == 0 &&
                         ((uintptr_t)v_cache % 16) == 0;
+    if (gather && threads < WAVES * 64) threads = WAVES * 64;
     const int64_t gather_v = gather ? (tokens + 8 * WAVES - 1) / (8 * WAVES) * kv_heads : 0;
-    if (tokens + gather_v > 0x7fffffff) return ERR_BAD_SHAPE;
-    auto kernel = qkv_row_post_kernel<bf16, 8>;
-    if (lds > 65536 - 64 && hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
+    // many tokens: a workgroup takes several, so that gains and biases are fetched once for them
+    const int per = tokens >= 1024 ? 4 : tokens >= 512 ? 2 : 1;
+    const int64_t blocks = (tokens + per - 1) / per;
+    if (blocks + gather_v > 0x7fffffff) return ERR_BAD_SHAPE;
+    const size_t rows = rot && style == 0 ? lds : 0;
+    auto kernel = iters == 1 ? qkv_row_post_vec_kernel<1> : qkv_row_post_vec_kernel<2>;
+    if (rows > 65536 - 512 && hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)rows) != hipSuccess)
       return ERR_LAUNCH;
-    kernel<<<(unsigned)(tokens + gather_v), 256, lds, stream>>>(
+    kernel<<<(unsigned)(blocks + gather_v), threads, rows, stream>>>(
         (bf16*)qkv, ld, q_off, k_off, v_off, q_gain, k_gain, eps, positions, cos_sin, rot, style, (bf16*)k_cache, (bf16*)v_cache,
-        slot_mapping, heads, kv_heads, head_dim, page_size, v_dim, bias, (int)tokens, (int)gather_v, mix);
+        slot_mapping, heads, kv_heads, head_dim, page_size, v_dim, bias, (int)tokens, per, (int)blocks, (int)gather_v, mix);
     return launch_status();
   }
   DINFER_DISPATCH_DTYPE(dtype, {
-    auto kernel = qkv_row_post_kernel<S, 1>;
+    auto kernel = qkv_row_post_kernel<S>;
     if (lds > 65536 - 64 && hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
       return ERR_LAUNCH;
     kernel<<<(unsigned)tokens, 256, lds, stream>>>((S*)qkv, ld, q_off, k_off, v_off, q_gain, k_gain, eps, positions, cos_sin, rot,
                                                    style, (S*)k_cache, (S*)v_cache, slot_mapping, heads, kv_heads, head_dim,
-                                                   page_size, v_dim, bias, (int)tokens, 0, mix);
+                                                   page_size, v_dim, bias, mix);
   });
   return launch_status();
 }
