@@ -88,18 +88,21 @@ __device__ __forceinline__ void gates(const Gru& p, const S* row, int c, const f
 }
 
 // A wave's tokens of a chunk: their gates go through every lane's registers at once, then the map they make of S,
-// S -> m S + s. FULL: all WT of them; else the first n, and the others change nothing (a = 0).
+// S -> m S + s. FULL: all WT of them; else the first n (the row `first` exists
+// whatever n is), and the others change nothing (a = 0).
 template <class S, int P, bool FULL>
 __device__ __forceinline__ void wave_tokens(const Gru& p, int64_t first, int n, int c, const float (&bz)[P], const float (&bx)[P],
                                             float (&a)[WT][P], float (&ac)[WT][P], float (&m)[P], float (&s)[P]) {
   const S* row = (const S*)p.proj + first * p.ld;
 #pragma unroll
   for (int t = 0; t < WT; ++t) {
-    if (FULL || t < n) {
-      gates<S, P>(p, row + (int64_t)t * p.ld, c, bz, bx, a[t], ac[t]);
-    } else {
+    gates<S, P>(p, row + (FULL || t < n ? (int64_t)t * p.ld : 0), c, bz, bx, a[t], ac[t]);
+    if (!FULL) {
 #pragma unroll
-      for (int e = 0; e < P; ++e) a[t][e] = ac[t][e] = 0.f;
+      for (int e = 0; e < P; ++e) {
+        a[t][e] = t < n ? a[t][e] : 0.f;
+        ac[t][e] = t < n ? ac[t][e] : 0.f;
+      }
     }
   }
 #pragma unroll
@@ -180,7 +183,7 @@ __device__ __forceinline__ void min_gru_wave(const Gru& p, S* __restrict__ out, 
 #pragma unroll
     for (int e = 0; e < P; ++e) g[t][e] = x.v[e];
   }
-  wave_tokens<S, P, FULL>(p, first, left, c, bz, bx, a, ac, m, sw);
+  wave_tokens<S, P, FULL>(p, left > 0 ? first : t0, left, c, bz, bx, a, ac, m, sw);
 #pragma unroll
   for (int e = 0; e < P; ++e) {
     ms[wave][0][lane * P + e] = m[e];
