@@ -242,7 +242,8 @@ class Attention(Mixer):
             self.kept_values = kept if self.value_mix == "mix" else None
         self.attn_buf = ws.buffer("attn", self.heads * self.v_dim)
         self.out_buf = ws.buffer("mixer_out", self.hidden)
-        self.attn_ws = attn_kernels.Workspace(ctx, self.heads, self.kv_heads, self.head_dim)
+        # (a layer with options runs the kernels with options, which need no scratch; nothing of the others is compiled for it)
+        self.attn_ws = None if self.extended else attn_kernels.Workspace(ctx, self.heads, self.kv_heads, self.head_dim)
 
     def forward(self, x, batch, cache: CacheView, into=None):
         T = batch.num_tokens
