@@ -389,17 +389,17 @@ def test_flash_kernel_with_values_of_another_size(case):
     assert err < 4e-2 * max(1.0, want.abs().max().item()), f"{case}: {err}"
 
 
-@pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("case", [(4, 2, 16, 24, 8, 1, 4), (3, 1, 20, 10, 20, 1, 8), (4, 2, 64, 64, 32, 1, 16), (4, 2, 64, 32, 64, 0, 16),
-                                  (2, 2, 24, 12, 0, 0, 8), (40, 8, 128, 128, 128, 1, 16), (80, 8, 128, 64, 128, 0, 16)])
-@pytest.mark.parametrize("T", [3, 70, 1100])
+ROWS = [(4, 2, 16, 24, 8, 1, 4), (3, 1, 20, 10, 20, 1, 8), (4, 2, 64, 64, 32, 1, 16), (4, 2, 64, 32, 64, 0, 16), (2, 2, 24, 12, 0, 0, 8),
+        (40, 8, 128, 128, 128, 1, 16), (80, 8, 128, 64, 128, 0, 16)]      # heads, kv heads, key and value sizes, rotated, pairing, page
+
+
+@pytest.mark.parametrize("case,T,dtype", [(c, T, dt) for c in ROWS[:6] for T in (3, 70) for dt in DTYPES]
+                         + [(c, 1100, "bfloat16") for c in ROWS if c[0] >= 4])
 def test_step_before_the_cache_with_whole_row_norms(case, T, dtype):
     """Norms over all heads at once, biases, both pairings, part of a head rotated, values mixed, keys and values in their
     pages (prompt portions that start anywhere, one row with no slot)."""
     from dinfer_amd.kernels import ops
     H, G, D, V, rot, style, page = case
-    if T > 100 and (H < 4 or dtype == "float32") or T < 100 and H > 40:
-        pytest.skip("covered by the other cases")
     dt = getattr(torch, dtype)
     g = torch.Generator().manual_seed(T + D)
     nq, nk, nv = H * D, G * D, G * V
