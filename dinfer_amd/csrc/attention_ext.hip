@@ -99,22 +99,24 @@ extern "C" int dinfer_attn_flash_ext_supports(int head_dim, int v_dim, int page_
 // Keys below keep_first stay visible behind the window; sinks [heads] float (or null) join the denominator; slope_exp E
 // takes 2^(-E (h + 1) / heads) times the distance off the scores; the output is multiplied by out_scale. v_dim: the size of
 // a value head (0: head_dim); out holds head h at column h v_dim. sigmoid_bias (or null): [heads] float, the weights are
-// sigmoid(score + bias), not normalised (no sinks then).
+// sigmoid(score + bias), not normalised (no sinks then). softcap C > 0: the scores are C tanh(scale q . k / C) (softmax
+// weights only); chunk N > 0: a row sees the keys of its own chunk of N positions only (counted from 0).
 extern "C" int dinfer_attn_flash_ext(const void* q, int64_t ld_q, void* out, int64_t ld_out, const void* k_cache,
                                      const void* v_cache, const int32_t* block_table, int64_t max_blocks,
                                      const int32_t* cu_seqlens, const int32_t* seq_lens, int num_reqs, int max_q_len,
                                      float scale, int window, int keep_first, const float* sinks, float slope_exp,
                                      float out_scale, int heads, int kv_heads, int head_dim, int v_dim, int page_size,
-                                     const float* sigmoid_bias, hipStream_t stream) {
+                                     const float* sigmoid_bias, float softcap, int chunk, hipStream_t stream) {
   if (num_reqs <= 0 || max_q_len <= 0) return OK;
   if (v_dim <= 0) v_dim = head_dim;
-  if (!dinfer_attn_flash_ext_supports(head_dim, v_dim, page_size, heads, kv_heads, sigmoid_bias ? 1 : 0) || (sigmoid_bias && sinks))
+  if (!dinfer_attn_flash_ext_supports(head_dim, v_dim, page_size, heads, kv_heads, sigmoid_bias ? 1 : 0) || (sigmoid_bias && (sinks || softcap > 0.f)))
     return ERR_UNSUPPORTED;
-  if (window < 0 || keep_first < 0 || !(scale > 0.f) || max_blocks <= 0 || ld_q % 8 || ld_out % 4 || !aligned16(q) ||
+  if (window < 0 || keep_first < 0 || chunk < 0 || !(softcap >= 0.f) || !(scale > 0.f) || max_blocks <= 0 || ld_q % 8 || ld_out % 4 || !aligned16(q) ||
       !aligned16(k_cache) || !aligned16(v_cache) || ((uintptr_t)out % 8))
     return ERR_BAD_SHAPE;
   const Args p{(const bf16*)q, ld_q, (bf16*)out, ld_out, (const bf16*)k_cache, (const bf16*)v_cache, block_table, max_blocks,
                cu_seqlens, seq_lens, num_reqs, max_q_len, window, heads, kv_heads, page_size,
-               FlashExt{keep_first, sinks, slope_exp, out_scale, scale, sigmoid_bias}};
+               FlashExt{keep_first, sinks, slope_exp, out_scale, softcap > 0.f ? 1.f : scale, sigmoid_bias, softcap,
+                        softcap > 0.f ? 2.f * LOG2E * scale / softcap : 0.f, chunk}};
   return sigmoid_bias ? launch_keys<SIGMOID>(head_dim, v_dim, p, stream) : launch_keys<OPTIONS>(head_dim, v_dim, p, stream);
 }

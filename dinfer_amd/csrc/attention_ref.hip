@@ -16,7 +16,9 @@
 //   v_dim          the value size where it differs from the key size;
 //   values in the key pages (v_cache null): a layer whose values are its keys stores them once;
 //   out_scale      o is multiplied by it on store;
-//   sigmoid_bias   one float a query head: no softmax, P_j = sigmoid(s_j + bias_h), not normalised over the keys.
+//   sigmoid_bias   one float a query head: no softmax, P_j = sigmoid(s_j + bias_h), not normalised over the keys;
+//   softcap C      s_j = C tanh(scale <q, k_j> / C) (before the distance bias);
+//   chunk N        positions fall into chunks of N, counted from 0, and a key of an earlier chunk is not seen.
 //
 // K and V are read from the cache pages through the request's block table
 // (K page [Hkv][ceil(D / 8)][page][8], V page [Hkv][D][page]); the step's own tokens were
@@ -40,7 +42,7 @@ __global__ void __launch_bounds__(WAVES * 64) attn_paged_ref_kernel(
     const S* __restrict__ v_cache, const int32_t* __restrict__ block_table, int64_t max_blocks,
     const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ seq_lens, int num_reqs, float scale,
     int window, int H, int Hkv, int D, int page, int keep_first, const float* __restrict__ sinks, float slope_exp,
-    int Dv, float out_scale, const float* __restrict__ sigmoid_bias) {
+    int Dv, float out_scale, const float* __restrict__ sigmoid_bias, float softcap, int chunk) {
   __shared__ float qs[WAVES][MAX_D];
   __shared__ float ps[WAVES][64];
   const int t = blockIdx.x;
@@ -57,7 +59,8 @@ __global__ void __launch_bounds__(WAVES * 64) attn_paged_ref_kernel(
   const int b = lo_b;
   const int q_len = cu_seqlens[b + 1] - cu_seqlens[b];
   const int p = seq_lens[b] - q_len + (t - cu_seqlens[b]);
-  const int first_key = window > 0 ? (p - window + 1 > 0 ? p - window + 1 : 0) : 0;
+  int first_key = window > 0 ? (p - window + 1 > 0 ? p - window + 1 : 0) : 0;
+  if (chunk > 0) first_key = max(first_key, p - p % chunk);
   const int32_t* bt = block_table + (int64_t)b * max_blocks;
   const int hk = live ? h / (H / Hkv) : 0;
   const int Dp = (D + 7) & ~7;  // a head's keys fill whole 8-entry pieces of a page (the last one padded)
@@ -88,7 +91,9 @@ __global__ void __launch_bounds__(WAVES * 64) attn_paged_ref_kernel(
       const int off = j % page;
       float acc = 0.f;
       for (int d = 0; d < D; ++d) acc += qs[wave][d] * to_f32(kr[k_page_offset(off, d, page)]);
-      s = acc * scale - slope * (float)(p - j);
+      s = acc * scale;
+      if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+      s -= slope * (float)(p - j);
     }
     float pj, alpha = 1.f;
     if (sigmoid_bias) {
@@ -298,7 +303,7 @@ extern "C" int dinfer_attn_paged_ref(int dtype, const void* q, int64_t ld_q, voi
   DINFER_DISPATCH_DTYPE(dtype, {
     attn_paged_ref_kernel<S><<<grid, WAVES * 64, 0, stream>>>(
         (const S*)q, ld_q, (S*)out, ld_out, (const S*)k_cache, (const S*)v_cache, block_table, max_blocks, cu_seqlens,
-        seq_lens, num_reqs, scale, window, heads, kv_heads, head_dim, page_size, 0, nullptr, 0.f, head_dim, 1.f, nullptr);
+        seq_lens, num_reqs, scale, window, heads, kv_heads, head_dim, page_size, 0, nullptr, 0.f, head_dim, 1.f, nullptr, 0.f, 0);
   });
   return launch_status();
 }
@@ -310,19 +315,20 @@ extern "C" int dinfer_attn_paged_ext(int dtype, const void* q, int64_t ld_q, voi
                                      int64_t max_blocks, const int32_t* cu_seqlens, const int32_t* seq_lens,
                                      int num_reqs, int64_t tokens, float scale, int window, int keep_first,
                                      const float* sinks, float slope_exp, int heads, int kv_heads, int head_dim,
-                                     int v_dim, int page_size, float out_scale, const float* sigmoid_bias,
-                                     hipStream_t stream) {
+                                     int v_dim, int page_size, float out_scale, const float* sigmoid_bias, float softcap,
+                                     int chunk, hipStream_t stream) {
   if (tokens <= 0 || num_reqs <= 0) return OK;
   if (heads <= 0 || kv_heads <= 0 || heads % kv_heads != 0 || head_dim <= 0 || v_dim <= 0 || page_size <= 0 ||
-      max_blocks <= 0 || window < 0 || keep_first < 0 || tokens > 0x7fffffff || (!v_cache && v_dim != head_dim))
+      max_blocks <= 0 || window < 0 || keep_first < 0 || chunk < 0 || !(softcap >= 0.f) || tokens > 0x7fffffff ||
+      (!v_cache && v_dim != head_dim))
     return ERR_BAD_SHAPE;
   if (head_dim > MAX_D || v_dim > MAX_D || (sigmoid_bias && sinks)) return ERR_UNSUPPORTED;
   const dim3 grid((unsigned)tokens, (unsigned)((heads + WAVES - 1) / WAVES));
   DINFER_DISPATCH_DTYPE(dtype, {
     attn_paged_ref_kernel<S><<<grid, WAVES * 64, 0, stream>>>(
         (const S*)q, ld_q, (S*)out, ld_out, (const S*)k_cache, (const S*)v_cache, block_table, max_blocks, cu_seqlens,
-        seq_lens, num_reqs, scale, window, heads, kv_heads, head_dim, page_size, window > 0 ? keep_first : 0, sinks,
-        slope_exp, v_dim, out_scale, sigmoid_bias);
+        seq_lens, num_reqs, scale, window, heads, kv_heads, head_dim, page_size, window > 0 || chunk > 0 ? keep_first : 0,
+        sinks, slope_exp, v_dim, out_scale, sigmoid_bias, softcap, chunk);
   });
   return launch_status();
 }

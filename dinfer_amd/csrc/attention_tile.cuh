@@ -23,8 +23,9 @@
 // Options of the flash kernel (KIND other than PLAIN; dinfer_attn_flash_ext, which serves single rows as well): the first
 // keep_first keys stay visible behind the window (one more short run of key blocks, walked by wave 0); a sink a head joins
 // the softmax's denominator when the waves' parts are combined; 2^(-slope_exp (h + 1) / H) times the distance is taken off
-// the scores (in raw score units, before the maximum); the output is multiplied by out_scale; or (SIGMOID) the weights are
-// sigmoids of the scores plus a bias a head, and nothing is normalised.
+// the scores (in raw score units, before the maximum); the scores are capped, C tanh(s / C), and a query sees only the keys
+// of its own chunk of positions (a lower bound a row, like a window's); the output is multiplied by out_scale; or (SIGMOID)
+// the weights are sigmoids of the scores plus a bias a head, and nothing is normalised.
 #pragma once
 #include "common.cuh"
 
@@ -114,6 +115,7 @@ struct Tile {
   float bias_log2e = 0.f;  // SIGMOID: the head's bias in base-2 units
   int keep_first = 0;      // EXT: keys below this stay visible whatever col_lo says
   float slope_raw = 0.f;   // EXT: taken off a raw score per key of distance (the slope divided by the scale)
+  float cap = 0.f, cap_in = 0.f;   // OPTIONS: scores become cap tanh(.), cap_in = 2 log2(e) scale / cap (0: no cap)
   static constexpr float LAZY = 6.f;       // weights up to 2^6 before the reference follows the maximum
   f32x4 o[NT][DV];
   float m[NT], l[NT];
@@ -228,6 +230,12 @@ struct Tile {
       for (int r = 0; r < 4; ++r) {
         x[r] = s[t][0][r];
         x[4 + r] = s[t][1][r];
+      }
+      if constexpr (KIND == OPTIONS) {
+        if (cap_in != 0.f) {     // (uniform) tanh y = 1 - 2 / (1 + e^2y); what follows takes scores in units of one
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[e] = fmaf(-2.f * cap, __builtin_amdgcn_rcpf(1.f + exp2_raw(cap_in * x[e])), cap);
+        }
       }
       if (EXT) {
         const float far = (float)(col_hi[t] - 1 - kg);   // the distance of the lane's first key from the column's position
@@ -363,8 +371,10 @@ struct FlashExt {
   const float* sinks;   // [H] float or null
   float slope_exp;      // 0: no distance bias
   float out_scale;
-  float scale;          // the score scale itself (scale_log2e / log2(e))
+  float scale;          // the score scale itself (scale_log2e / log2(e)); with a cap: 1, the scale is in cap_in
   const float* biases;  // SIGMOID: [H] float, added to the scores
+  float cap, cap_in;    // softly capped scores (cap_in 0: none)
+  int chunk;            // > 0: keys of the row's own chunk of positions only
 };
 
 template <int DT, int QT, bool P2, int KIND = PLAIN, int DV = DT>
@@ -403,6 +413,14 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 8))
   if (skip_single && q_len == 1) return;  // single rows go to the split-K kernel
   const int32_t* bt = block_table + (int64_t)b * max_blocks;
 
+  // the first key (but for kept ones) that the row at a position sees
+  auto low_of = [&](int pos) {
+    int lo = window > 0 ? (pos - window + 1 > 0 ? pos - window + 1 : 0) : 0;
+    if constexpr (EXT) {
+      if (ext.chunk > 0) lo = max(lo, pos - pos % ext.chunk);
+    }
+    return lo;
+  };
   bf16x8 qf[QT][KS];
   int col_lo[QT], col_hi[QT];
 #pragma unroll
@@ -417,13 +435,13 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 8))
     }
     const int pos = hist + rc;
     col_hi[t] = pos + 1;
-    col_lo[t] = window > 0 ? (pos - window + 1 > 0 ? pos - window + 1 : 0) : 0;
+    col_lo[t] = low_of(pos);
   }
   // the keys any row of the tile sees, and this wave's run of 32-key blocks among them
   const int p_first = hist + q0;
   const int p_last = hist + (q0 + QW < q_len ? q0 + QW : q_len) - 1;
   const int all_hi = p_last + 1;
-  const int all_lo = window > 0 ? (p_first - window + 1 > 0 ? p_first - window + 1 : 0) : 0;
+  const int all_lo = low_of(p_first), last_lo = low_of(p_last);
   const int blk_first = all_lo >> 5, blk_end = (all_hi + 31) >> 5;
   const int per = (blk_end - blk_first + 3) >> 2;
   const int blk0 = blk_first + wave * per;
@@ -434,12 +452,14 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 8))
   Tile<DT, QT, P2, KIND, DV> tl;
   tl.init(kc, vc, bt, (int)max_blocks, hk, Hkv, ps, k_lo, k_hi, scale_log2e);
   if constexpr (EXT) {
-    tl.keep_first = window > 0 ? ext.keep_first : 0;
+    tl.keep_first = window > 0 || ext.chunk > 0 ? ext.keep_first : 0;
+    tl.cap = ext.cap;
+    tl.cap_in = ext.cap_in;
     tl.slope_raw = ext.slope_exp != 0.f ? exp2f(-ext.slope_exp * (float)(h + 1) / (float)H) / ext.scale : 0.f;
     if constexpr (KIND == SIGMOID) tl.bias_log2e = ext.biases[h] * LOG2E;
   }
   tl.template walk<true>(qf, col_lo, col_hi, [&](int kb) {
-    return kb + 31 > p_first || kb < all_lo || (window > 0 && kb < p_last - window + 1) || (EXT && kb + 32 > k_hi);
+    return kb + 31 > p_first || kb < all_lo || kb < last_lo || (EXT && kb + 32 > k_hi);
   });
   if constexpr (EXT) {
     // the kept first keys that the window of the tile's first row has passed: one more run, every block masked

@@ -42,6 +42,7 @@ __device__ __forceinline__ int request_of(const int32_t* __restrict__ cu, int nu
 }
 
 __device__ __forceinline__ float silu_f(float z) { return z / (1.f + expf(-z)); }
+__device__ __forceinline__ float gate_of(float z, int act) { return (act ? 1.f : z) / (1.f + expf(-z)); }   // sigmoid, else silu
 __device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
 // work row: q (H D) | k (H D) | v (H V), float; a thread an entry
@@ -391,14 +392,14 @@ __global__ void __launch_bounds__(256) gated_group_norm_kernel(const float* __re
                                                                const S* __restrict__ z, int64_t ld_z, int64_t z_off,
                                                                const float* __restrict__ w, S* __restrict__ out,
                                                                int64_t ld_out, int64_t col_off, int group, float eps,
-                                                               float out_scale, int gate_first) {
+                                                               float out_scale, int gate_first, int gate_act) {
   __shared__ float red[16];
   const int64_t t = blockIdx.x;
   const int c0 = blockIdx.y * group;
   auto value = [&](int c) {
     float u = y[t * ld_y + c];
     if (skip) u = __builtin_fmaf(skip[c / V], x[t * ld_x + c], u);
-    return gate_first ? u * silu_f(to_f32(z[t * ld_z + z_off + c])) : u;
+    return gate_first ? u * gate_of(to_f32(z[t * ld_z + z_off + c]), gate_act) : u;
   };
   float ss = 0.f;
   constexpr int KEEP = 4;                    // a group of up to 1,024 columns stays in registers between the two passes
@@ -422,7 +423,7 @@ __global__ void __launch_bounds__(256) gated_group_norm_kernel(const float* __re
       const int c = c0 + threadIdx.x + 256 * e;
       if (c < c0 + group) {
         float r = kept[e] * inv * (w ? w[c] : 1.f) * out_scale;
-        if (!gate_first) r *= silu_f(to_f32(z[t * ld_z + z_off + c]));
+        if (!gate_first) r *= gate_of(to_f32(z[t * ld_z + z_off + c]), gate_act);
         out[t * ld_out + col_off + c] = from_f32<S>(r);
       }
     }
@@ -430,8 +431,54 @@ __global__ void __launch_bounds__(256) gated_group_norm_kernel(const float* __re
   }
   for (int c = c0 + threadIdx.x; c < c0 + group; c += 256) {
     float r = value(c) * inv * (w ? w[c] : 1.f) * out_scale;
-    if (!gate_first) r *= silu_f(to_f32(z[t * ld_z + z_off + c]));
+    if (!gate_first) r *= gate_of(to_f32(z[t * ld_z + z_off + c]), gate_act);
     out[t * ld_out + col_off + c] = from_f32<S>(r);
+  }
+}
+
+// Groups of more than 256 columns, the gate after the norm, bf16 rows of whole 16-byte pieces: a thread keeps its pieces of 8
+// columns (ITERS of them) in registers between the two passes.
+template <int ITERS>
+__global__ void __launch_bounds__(256) gated_group_norm_regs_kernel(const float* __restrict__ y, int64_t ld_y,
+                                                                    const bf16* __restrict__ z, int64_t ld_z, int64_t z_off,
+                                                                    const float* __restrict__ w, bf16* __restrict__ out,
+                                                                    int64_t ld_out, int64_t col_off, int group, float eps,
+                                                                    float out_scale, int gate_act) {
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x;
+  const int c0 = blockIdx.y * group, n8 = group / 8;
+  f32x4 v[ITERS][2];
+  bf16x8 g[ITERS];
+  float ss = 0.f;
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int i = it * 256 + threadIdx.x;
+    if (i < n8) {
+      const int c = c0 + 8 * i;
+      v[it][0] = *(const f32x4*)(y + t * ld_y + c);
+      v[it][1] = *(const f32x4*)(y + t * ld_y + c + 4);
+      g[it] = *(const bf16x8*)(z + t * ld_z + z_off + c);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss = __builtin_fmaf(v[it][j >> 2][j & 3], v[it][j >> 2][j & 3], ss);
+    }
+  }
+  const float inv = out_scale / sqrtf(block_sum(ss, red) / (float)group + eps);
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int i = it * 256 + threadIdx.x;
+    if (i < n8) {
+      const int c = c0 + 8 * i;
+      f32x4 a = {1.f, 1.f, 1.f, 1.f}, b = a;
+      if (w) {
+        a = *(const f32x4*)(w + c);
+        b = *(const f32x4*)(w + c + 4);
+      }
+      bf16x8 r;
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        r[j] = (bf16)(v[it][j >> 2][j & 3] * inv * (j < 4 ? a[j & 3] : b[j & 3]) * gate_of((float)g[it][j], gate_act));
+      *(bf16x8*)(out + t * ld_out + col_off + c) = r;
+    }
   }
 }
 
@@ -444,7 +491,8 @@ __global__ void __launch_bounds__(256) gated_group_norm_wave_kernel(const float*
                                                                     const S* __restrict__ z, int64_t ld_z, int64_t z_off,
                                                                     const float* __restrict__ w, S* __restrict__ out,
                                                                     int64_t ld_out, int64_t col_off, int groups, int group,
-                                                                    float eps, float out_scale, int gate_first) {
+                                                                    float eps, float out_scale, int gate_first,
+                                                                    int gate_act) {
   const int64_t t = blockIdx.x;
   const int g = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (g >= groups) return;                   // (a whole wave leaves: the shuffles below see full waves only)
@@ -460,7 +508,7 @@ __global__ void __launch_bounds__(256) gated_group_norm_wave_kernel(const float*
       const int c = c0 + i;
       float u = y[t * ld_y + c];
       if (skip) u = __builtin_fmaf(skip[c / V], x[t * ld_x + c], u);
-      gate[e] = silu_f(to_f32(z[t * ld_z + z_off + c]));
+      gate[e] = gate_of(to_f32(z[t * ld_z + z_off + c]), gate_act);
       kept[e] = gate_first ? u * gate[e] : u;
     }
     ss = __builtin_fmaf(kept[e], kept[e], ss);
@@ -567,28 +615,42 @@ extern "C" int dinfer_decay_recurrence(const float* q, int64_t ldq, const float*
   return launch_status();
 }
 
-// y [T, ld_y] float, `groups` groups of `group` columns each; x [T, ld_x] float with skip [groups * group / V] (both or
+// gate_act: 0 silu, 1 sigmoid. y [T, ld_y] float, `groups` groups of `group` columns each; x [T, ld_x] float with skip [groups * group / V] (both or
 // neither); z [T, ld_z] in the step's dtype, the gate's columns from z_off; w [groups * group] float or null.
 extern "C" int dinfer_gated_group_norm(int dtype, const float* y, int64_t ld_y, const float* x, int64_t ld_x,
                                        const float* skip, int V, const void* z, int64_t ld_z, int64_t z_off,
                                        const float* w, void* out, int64_t ld_out, int64_t col_off, int64_t tokens,
-                                       int groups, int group, float eps, float out_scale, int gate_first,
+                                       int groups, int group, float eps, float out_scale, int gate_first, int gate_act,
                                        hipStream_t stream) {
   if (tokens <= 0) return OK;
   if (groups <= 0 || group <= 0 || groups > 65535 || tokens > 0x7fffffff || (skip && (!x || V <= 0))) return ERR_BAD_SHAPE;
+  if (gate_act != 0 && gate_act != 1) return ERR_UNSUPPORTED;
+  if (dtype == DT_BF16 && !skip && !gate_first && group > 256 && group % 8 == 0 && group <= 256 * 8 * 4 && ld_y % 4 == 0 &&
+      ld_z % 8 == 0 && z_off % 8 == 0 && ld_out % 8 == 0 && col_off % 8 == 0 && ((uintptr_t)y % 16) == 0 &&
+      ((uintptr_t)z % 16) == 0 && ((uintptr_t)w % 16) == 0 && ((uintptr_t)out % 16) == 0) {
+    const dim3 rgrid((unsigned)tokens, (unsigned)groups);
+#define DINFER_GROUP_REGS(IT)                                                                                           \
+  gated_group_norm_regs_kernel<IT><<<rgrid, 256, 0, stream>>>(y, ld_y, (const bf16*)z, ld_z, z_off, w, (bf16*)out, ld_out, \
+                                                              col_off, group, eps, out_scale, gate_act)
+    if (group <= 256 * 8) DINFER_GROUP_REGS(1);
+    else if (group <= 256 * 8 * 2) DINFER_GROUP_REGS(2);
+    else DINFER_GROUP_REGS(4);
+#undef DINFER_GROUP_REGS
+    return launch_status();
+  }
   if (group <= 256) {
     const dim3 wgrid((unsigned)tokens, (unsigned)((groups + 3) / 4));
     DINFER_DISPATCH_DTYPE(dtype, {
       gated_group_norm_wave_kernel<S><<<wgrid, 256, 0, stream>>>(y, ld_y, x, ld_x, skip, V, (const S*)z, ld_z, z_off, w,
                                                                 (S*)out, ld_out, col_off, groups, group, eps, out_scale,
-                                                                gate_first);
+                                                                gate_first, gate_act);
     });
     return launch_status();
   }
   const dim3 grid((unsigned)tokens, (unsigned)groups);
   DINFER_DISPATCH_DTYPE(dtype, {
     gated_group_norm_kernel<S><<<grid, 256, 0, stream>>>(y, ld_y, x, ld_x, skip, V, (const S*)z, ld_z, z_off, w, (S*)out,
-                                                         ld_out, col_off, group, eps, out_scale, gate_first);
+                                                         ld_out, col_off, group, eps, out_scale, gate_first, gate_act);
   });
   return launch_status();
 }

@@ -2,14 +2,16 @@
 //
 // Two ways of naming the groups:
 //   heads    group z is a head: A_z, W_z and C_z are column blocks / slabs at fixed strides (a_zs, w_zs, c_zs) and all
-//            groups have the same M rows. With `gate`, row m of C_z is multiplied by sigmoid(gate[m, z]).
+//            groups have the same M rows. With `gate`, row m of C_z is multiplied by sigmoid(gate[m, z]), or entry by entry
+//            by sigmoid(gate[m, z N + n]).
 //   experts  group g is an expert: its rows are the entries offsets[g] .. offsets[g+1] of a list sorted by expert
 //            (`perm`: sorted place -> entry = token * top + choice). A row is read either from the entry's token
 //            (a_div = top: the gate and up projections read the step's rows) or from the sorted place itself
 //            (a_div = 0: the down projection reads what the first product left), and written to the sorted place
 //            or, with c_to_perm, to the entry. The work list `tiles` names (expert, first sorted place) of every
 //            row tile; entries beyond the step's tiles hold -1 and their workgroups leave at once.
-// GATED: W_g = [gate rows; up rows] stacked, gate_n rows each, and C = silu(A Wgate^T) * (A Wup^T).
+// GATED: W_g = [gate rows; up rows] stacked, gate_n rows each, and C = silu(A Wgate^T) * (A Wup^T), or with clamps, from
+// g = min(A Wgate^T, limit) and u = A Wup^T clamped to [-limit, limit]: C = g sigmoid(slope g) (u + 1).
 // row_scale (experts): the row of A belonging to entry e is multiplied by row_scale[e]; the product being linear in it, the
 // float sums are, before the activation.
 //
@@ -41,10 +43,12 @@ struct Groups {
   int a_div;                // experts: > 0: A row = perm[i] / a_div; 0: A row = i
   int c_to_perm;            // experts: C row = perm[i] instead of i
   const void* gate; int64_t ld_gate;   // heads: optional
+  int gate_entries;         // heads: the gate has a column an entry of C's rows (else one a head)
   int gate_n;               // GATED: rows of each half of W_g
   int tm;                   // rows of a tile: 64 on the vector ALUs, 16 or 128 on the matrix cores
   int act;                  // not GATED: 0 nothing, 1 silu, 2 gelu (error function), 3 the square of relu on every result
   const float* row_scale;   // experts: a factor an entry on its row of A, or null
+  int clamped; float limit, slope;     // GATED: the form with clamps
 };
 
 __device__ __forceinline__ float silu(float x) { return x / (1.f + expf(-x)); }
@@ -54,6 +58,18 @@ __device__ __forceinline__ float plain_act(float x, int act) {
   if (act == 2) return 0.5f * x * (1.f + erff(x * 0.7071067811865476f));
   if (act == 3) return x > 0.f ? x * x : 0.f;
   return x;
+}
+
+__device__ __forceinline__ float gated_value(const Groups& p, float g, float u) {
+  if (!p.clamped) return silu(g) * u;
+  g = fminf(g, p.limit);
+  u = fminf(fmaxf(u, -p.limit), p.limit);
+  return g * sigmoid(p.slope * g) * (u + 1.f);
+}
+// what entry n of row `row` of head z's block is multiplied by
+template <class S>
+__device__ __forceinline__ float head_gate(const Groups& p, int64_t row, int z, int n) {
+  return p.gate ? sigmoid(to_f32(((const S*)p.gate)[row * p.ld_gate + (p.gate_entries ? (int64_t)z * p.N + n : z)])) : 1.f;
 }
 
 constexpr int BM = 64, BN = 64, BK = 16;
@@ -146,15 +162,14 @@ __global__ void __launch_bounds__(256) grouped_valu_kernel(Groups p) {
     const int r = ty * 4 + i;
     if (r >= tl.rows) continue;
     const int64_t cr = tl.c_row(r);
-    float g = 1.f;
-    if (p.gate) g = sigmoid(to_f32(((const S*)p.gate)[cr * p.ld_gate + tl.z]));
+    const float g1 = p.gate_entries ? 1.f : head_gate<S>(p, cr, tl.z, 0);
     const float rs = tl.scale_of(p, r);
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int gn = n0 + tx * 4 + j;
       if (gn < p.N) {
-        float v = GATED ? silu(acc[i][j] * rs) * (acu[i][j] * rs) : plain_act(acc[i][j] * rs, p.act);
-        C[cr * p.ldc + gn] = from_f32<O>(v * g);
+        const float v = GATED ? gated_value(p, acc[i][j] * rs, acu[GATED ? i : 0][j] * rs) : plain_act(acc[i][j] * rs, p.act);
+        C[cr * p.ldc + gn] = from_f32<O>(v * (p.gate_entries ? head_gate<S>(p, cr, tl.z, gn) : g1));
       }
     }
   }
@@ -259,15 +274,14 @@ __global__ void __launch_bounds__(256) grouped_mfma_big_kernel(Groups p) {
       const int row = wm * 64 + i * 16 + kq * 4 + r;
       if (row >= tl.rows) continue;
       const int64_t cr = tl.c_row(row);
-      float g = 1.f;
-      if (p.gate) g = sigmoid((float)((const bf16*)p.gate)[cr * p.ld_gate + tl.z]);
+      const float g1 = p.gate_entries ? 1.f : head_gate<bf16>(p, cr, tl.z, 0);
       const float rs = tl.scale_of(p, row);
 #pragma unroll
       for (int j = 0; j < (GATED ? 2 : 4); ++j) {
         const int gn = GATED ? n0 + wn * 32 + j * 16 + lr : n0 + wn * 64 + j * 16 + lr;
         if (gn < p.N) {
-          const float v = GATED ? silu(acc[i][j][r] * rs) * (acc[i][j + 2][r] * rs) : plain_act(acc[i][j][r] * rs, p.act);
-          C[cr * p.ldc + gn] = from_f32<O>(v * g);
+          const float v = GATED ? gated_value(p, acc[i][j][r] * rs, acc[i][(j + 2) & 3][r] * rs) : plain_act(acc[i][j][r] * rs, p.act);
+          C[cr * p.ldc + gn] = from_f32<O>(v * (p.gate_entries ? head_gate<bf16>(p, cr, tl.z, gn) : g1));
         }
       }
     }
@@ -328,11 +342,10 @@ __global__ void __launch_bounds__(256) grouped_mfma_small_kernel(Groups p) {
     if (GATED) u += part[w][GATED ? 1 : 0][row][col];
   }
   const int64_t cr = tl.c_row(row);
-  float g = 1.f;
-  if (p.gate) g = sigmoid((float)((const bf16*)p.gate)[cr * p.ld_gate + tl.z]);
+  const float g = head_gate<bf16>(p, cr, tl.z, n0 + col);
   O* C = (O*)p.C + (experts ? 0 : (int64_t)tl.z * p.c_zs);
   const float rs = tl.scale_of(p, row);
-  C[cr * p.ldc + n0 + col] = from_f32<O>((GATED ? silu(v * rs) * (u * rs) : plain_act(v * rs, p.act)) * g);
+  C[cr * p.ldc + n0 + col] = from_f32<O>((GATED ? gated_value(p, v * rs, u * rs) : plain_act(v * rs, p.act)) * g);
 }
 
 // ---- routing ---------------------------------------------------------------------------------------------------
@@ -608,15 +621,17 @@ int launch_groups(int dtype, Groups p, unsigned gy, unsigned gz, hipStream_t str
 
 }  // namespace
 
-// C[m, z*c_zs + n] = (sigmoid(gate[m, z]) *) sum_k A[m, z*a_zs + k] W[z*w_zs + n*ldw + k], z < groups.
+// C[m, z*c_zs + n] = (sigmoid(gate[m, z]) *) sum_k A[m, z*a_zs + k] W[z*w_zs + n*ldw + k], z < groups. gate_entries: the
+// gate's column is z*N + n instead of z.
 extern "C" int dinfer_heads_nt(int dtype, const void* A, int64_t lda, int64_t a_zs, const void* W, int64_t ldw,
                                int64_t w_zs, void* C, int64_t ldc, int64_t c_zs, int64_t M, int64_t N, int64_t K,
-                               int64_t groups, const void* gate, int64_t ld_gate, hipStream_t stream) {
+                               int64_t groups, const void* gate, int64_t ld_gate, int gate_entries, hipStream_t stream) {
   if (M <= 0 || N <= 0 || groups <= 0) return OK;
   if (K <= 0 || ldw < K || M > 0x7fffffff || N > 0x7fffffff || K > 0x7fffffff || groups > 65535) return ERR_BAD_SHAPE;
   Groups p{};
   p.A = A; p.lda = lda; p.a_zs = a_zs; p.W = W; p.ldw = ldw; p.w_zs = w_zs; p.C = C; p.ldc = ldc; p.c_zs = c_zs;
   p.M = (int)M; p.N = (int)N; p.K = (int)K; p.gate = gate; p.ld_gate = ld_gate;
+  p.gate_entries = gate && gate_entries;
   p.tm = !mfma_fits(dtype, p) ? BM : M <= TM_SMALL ? TM_SMALL : TM_BIG;
   const int64_t gy = (M + p.tm - 1) / p.tm;
   if (gy > 65535) return ERR_UNSUPPORTED;
@@ -624,12 +639,12 @@ extern "C" int dinfer_heads_nt(int dtype, const void* A, int64_t lda, int64_t a_
 }
 
 // The products of the experts (see the head of the file). W [experts][rows][ldw] with w_zs elements an expert;
-// gated 1: rows = 2 N (gate rows, then up rows); 0: plain; 2, 3, 4: plain with silu, gelu (error function) or the square of
+// gated 1: rows = 2 N (gate rows, then up rows), with clamps where limit > 0; 0: plain; 2, 3, 4: plain with silu, gelu (error function) or the square of
 // relu on every result. max_tiles: the length of `tiles`. row_scale (may be null): float, a factor an entry on its row of A.
 extern "C" int dinfer_experts_nt(int dtype, int gated, const void* A, int64_t lda, const void* W, int64_t ldw,
                                  int64_t w_zs, void* C, int64_t ldc, int64_t N, int64_t K, const int32_t* tiles,
                                  int64_t max_tiles, int tile_rows, const int32_t* offsets, const int32_t* perm, int a_div,
-                                 int c_to_perm, const float* row_scale, hipStream_t stream) {
+                                 int c_to_perm, const float* row_scale, float limit, float slope, hipStream_t stream) {
   if (N <= 0 || max_tiles <= 0) return OK;
   if (K <= 0 || ldw < K || lda < K || ldc < N || N > 0x7fffffff || K > 0x7fffffff || max_tiles > 65535 || !tiles ||
       !offsets || !perm || tile_rows <= 0)
@@ -639,6 +654,7 @@ extern "C" int dinfer_experts_nt(int dtype, int gated, const void* A, int64_t ld
   p.N = (int)N; p.K = (int)K; p.tiles = tiles; p.offsets = offsets; p.perm = perm; p.a_div = a_div;
   p.c_to_perm = c_to_perm; p.gate_n = (int)N; p.tm = tile_rows;
   p.row_scale = row_scale;
+  p.clamped = gated == 1 && limit > 0.f; p.limit = limit; p.slope = slope;
   if (gated < 0 || gated > 4) return ERR_UNSUPPORTED;
   p.act = gated >= 2 ? gated - 1 : 0;
   if (!mfma_fits(dtype, p) && tile_rows > BM) return ERR_UNSUPPORTED;

@@ -14,6 +14,8 @@
 //   chunks pass     what every chunk makes of S = 0, and the product of its decays (the portion's last chunk: nothing)
 //   scan            chunk by chunk, every entry of S by itself: a chunk's note becomes the S it starts from
 //   recurrence      as above, a chunk a workgroup, from that S; the portion's last chunk stores the request's state
+// With FIXED one constant decay a head takes the place of the decays a channel and token (lightning attention); then q, k
+// and v may pass a silu on their way in.
 // Chunks are counted from the portion's start. S is stored transposed, [slot][head][V][D]. A request whose step starts at
 // position 0 starts from S = 0, whatever its slot held.
 #include "common.cuh"
@@ -106,6 +108,8 @@ struct Gla {
   const int32_t* slots; const int32_t* cu; const int32_t* seq_lens;
   float* out; int64_t ld_out;
   int H, D, V, cl, vec;                               // vec: pieces of 8 operands come by 16-byte loads
+  const float* fixed;                                 // FIXED: [H], the head's decay
+  int act;                                            // 1: q, k and v are silu of what lies in memory
 };
 
 // where a chunk's note lies: places of different requests never meet (floor(cu / CL) + request grows by at least the
@@ -113,11 +117,11 @@ struct Gla {
 __device__ __forceinline__ int64_t place_of(int t0, int b, int chunk) { return (int64_t)(t0 / CL) + b + chunk; }
 
 // OUT: the recurrence itself; else the chunks pass. A thread owns RPT consecutive rows of CPT columns (D <= 32 RPT).
-template <class O, int RPT, int CPT, bool OUT>
+template <class O, int RPT, int CPT, bool OUT, bool FIXED>
 __global__ void __launch_bounds__(256) gla_kernel(Gla<O> p) {
   constexpr int DP = 32 * RPT, COLS = 8 * CPT;
   __shared__ __attribute__((aligned(16))) float ks[CH][DP];
-  __shared__ __attribute__((aligned(16))) float as[CH][DP];
+  __shared__ __attribute__((aligned(16))) float as[FIXED ? 1 : CH][DP];
   __shared__ __attribute__((aligned(16))) float qs[OUT ? CH : 1][DP];
   __shared__ __attribute__((aligned(16))) float vs[CH][COLS];
   // the request is the slowest index of the grid: the workgroups of one long request among many short ones then spread
@@ -170,7 +174,9 @@ __global__ void __launch_bounds__(256) gla_kernel(Gla<O> p) {
   // what a thread carries of the next 16 tokens: pieces of k, q and the decays, entries of v
   constexpr int PIECES = CH * DP / 8, NP = (PIECES + 255) / 256, NV = (CH * COLS + 255) / 256;
   Piece<O> pk[NP], pq[OUT ? NP : 1];
-  Piece<float> pa[NP];
+  Piece<float> pa[FIXED ? 1 : NP];
+  const float head_decay = FIXED ? p.fixed[h] : 1.f;
+  auto entry = [&](float x) { return p.act ? x / (1.f + expf(-x)) : x; };
   float pv[NV];
   auto piece = [&](auto& dst, const auto* src, bool in, int d) {
     if (!in) { dst.zero(); return; }
@@ -189,19 +195,22 @@ __global__ void __launch_bounds__(256) gla_kernel(Gla<O> p) {
       const int64_t t = t0 + ct + tok;
       piece(pk[e], p.k + t * p.ld + (int64_t)h * D + d, in, d);
       if constexpr (OUT) piece(pq[e], p.q + t * p.ld + (int64_t)h * D + d, in, d);
-      piece(pa[e], p.decay + t * p.ldd + (int64_t)h * D + d, in, d);
+      if constexpr (!FIXED) piece(pa[e], p.decay + t * p.ldd + (int64_t)h * D + d, in, d);
     }
 #pragma unroll
     for (int e = 0; e < NV; ++e) {
       const int idx = tid + e * 256;
       const int tok = idx / COLS, c = cb * COLS + idx % COLS;
-      pv[e] = (idx < CH * COLS && ct + tok < n && c < V) ? to_f32(p.v[(int64_t)(t0 + ct + tok) * p.ld + (int64_t)h * V + c]) : 0.f;
+      pv[e] = (idx < CH * COLS && ct + tok < n && c < V) ? entry(to_f32(p.v[(int64_t)(t0 + ct + tok) * p.ld + (int64_t)h * V + c])) : 0.f;
     }
   };
-  auto put = [&](float* dst, const auto& src, float f) {
+  auto put = [&](float* dst, const auto& src, float f, bool raw) {
     f32x4 a, b2;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) { a[i] = src.get(i) * f; b2[i] = src.get(4 + i) * f; }
+    for (int i = 0; i < 4; ++i) {
+      a[i] = (raw ? src.get(i) : entry(src.get(i))) * f;
+      b2[i] = (raw ? src.get(4 + i) : entry(src.get(4 + i))) * f;
+    }
     *(f32x4*)dst = a;
     *(f32x4*)(dst + 4) = b2;
   };
@@ -211,7 +220,7 @@ __global__ void __launch_bounds__(256) gla_kernel(Gla<O> p) {
 #pragma unroll
     for (int i = 0; i < RPT; ++i) {
       kk[i] = ks[tok][rg * RPT + i];
-      aa[i] = as[tok][rg * RPT + i];
+      aa[i] = FIXED ? head_decay : as[FIXED ? 0 : tok][rg * RPT + i];
       if constexpr (OUT) qq[i] = qs[tok][rg * RPT + i];
       else prod[i] *= aa[i];
     }
@@ -238,9 +247,9 @@ __global__ void __launch_bounds__(256) gla_kernel(Gla<O> p) {
       const int idx = tid + e * 256;
       if (idx < PIECES) {
         const int tok = idx / (DP / 8), d = (idx % (DP / 8)) * 8;
-        put(&ks[tok][d], pk[e], 1.f);
-        if constexpr (OUT) put(&qs[tok][d], pq[e], p.q_scale);
-        put(&as[tok][d], pa[e], 1.f);
+        put(&ks[tok][d], pk[e], 1.f, false);
+        if constexpr (OUT) put(&qs[tok][d], pq[e], p.q_scale, false);
+        if constexpr (!FIXED) put(&as[tok][d], pa[e], 1.f, true);
       }
     }
 #pragma unroll
@@ -348,16 +357,22 @@ __global__ void __launch_bounds__(256) gla_scan_kernel(Gla<O> p) {
   }
 }
 
-template <class O, int RPT>
+template <class O, int RPT, bool FIXED>
 void launch_gla(Gla<O> p, int64_t chunks, int num_reqs, bool wide, hipStream_t stream) {
   const auto grid = [&](int cols) { return dim3((unsigned)((p.V + cols - 1) / cols * p.H), (unsigned)chunks, (unsigned)num_reqs); };
   if (chunks > 1) {
-    gla_kernel<O, RPT, 2, false><<<grid(16), 256, 0, stream>>>(p);
+    gla_kernel<O, RPT, 2, false, FIXED><<<grid(16), 256, 0, stream>>>(p);
     const int64_t per = (int64_t)p.H * p.V * p.D;
     gla_scan_kernel<O><<<dim3((unsigned)((per + 255) / 256), 1, (unsigned)num_reqs), 256, 0, stream>>>(p);
   }
-  if (wide) gla_kernel<O, RPT, 2, true><<<grid(16), 256, 0, stream>>>(p);
-  else gla_kernel<O, RPT, 1, true><<<grid(8), 256, 0, stream>>>(p);
+  if (wide) gla_kernel<O, RPT, 2, true, FIXED><<<grid(16), 256, 0, stream>>>(p);
+  else gla_kernel<O, RPT, 1, true, FIXED><<<grid(8), 256, 0, stream>>>(p);
+}
+
+template <class O, int RPT>
+void pick_gla(const Gla<O>& p, int64_t chunks, int num_reqs, bool wide, hipStream_t stream) {
+  if (p.fixed) launch_gla<O, RPT, true>(p, chunks, num_reqs, wide, stream);
+  else launch_gla<O, RPT, false>(p, chunks, num_reqs, wide, stream);
 }
 
 }  // namespace
@@ -398,14 +413,17 @@ extern "C" int dinfer_channel_decay(int dtype, const void* proj, int64_t ld, int
 
 // q, k [T, H D], v [T, H V]: columns of rows of stride ld in the step's dtype; decay [T, ldd >= H D] float. state
 // [slots, H, V, D] float; out [T, ld_out] float, head h at column h V. cut: the step runs in chunks (dinfer_gla_cuts),
-// with notes [places, H, V, D] and products [places, H, D].
+// with notes [places, H, V, D] and products [places, H, D]. fixed [H] float in place of decay: one constant decay a head.
+// act 1: q, k and v are the silu of what the operands hold.
 extern "C" int dinfer_gla_recurrence(int dtype, const void* q, const void* k, const void* v, int64_t ld, const float* decay,
                                      int64_t ldd, float q_scale, float* state, float* notes, float* products,
                                      int64_t places, const int32_t* state_slots, const int32_t* cu_seqlens,
                                      const int32_t* seq_lens, float* out, int64_t ld_out, int num_reqs, int64_t tokens,
-                                     int64_t max_rows, int cut, int H, int D, int V, hipStream_t stream) {
+                                     int64_t max_rows, int cut, int H, int D, int V, const float* fixed, int act,
+                                     hipStream_t stream) {
   if (num_reqs <= 0 || max_rows <= 0) return OK;
-  if (H <= 0 || D <= 0 || V <= 0 || num_reqs > 65535 || ldd < (int64_t)H * D || ld_out < (int64_t)H * V || tokens > 0x7fffffff)
+  if ((decay == nullptr) == (fixed == nullptr) || (act && !fixed)) return ERR_BAD_SHAPE;
+  if (H <= 0 || D <= 0 || V <= 0 || num_reqs > 65535 || (decay && ldd < (int64_t)H * D) || ld_out < (int64_t)H * V || tokens > 0x7fffffff)
     return ERR_BAD_SHAPE;
   if (D > 256) return ERR_UNSUPPORTED;
   const int64_t chunks = cut ? (max_rows + CL - 1) / CL : 1;
@@ -416,12 +434,12 @@ extern "C" int dinfer_gla_recurrence(int dtype, const void* q, const void* k, co
     const bool vec = D % 8 == 0 && ((int64_t)ld * es) % 16 == 0 && ldd % 4 == 0 && ((uintptr_t)q % 16) == 0 &&
                      ((uintptr_t)k % 16) == 0 && ((uintptr_t)decay % 16) == 0;
     Gla<S> p{(const S*)q, (const S*)k, (const S*)v, ld, decay, ldd, q_scale, state, notes, products, state_slots, cu_seqlens,
-             seq_lens, out, ld_out, H, D, V, chunks > 1 ? CL : 0x40000000, vec ? 1 : 0};
+             seq_lens, out, ld_out, H, D, V, chunks > 1 ? CL : 0x40000000, vec ? 1 : 0, fixed, act};
     const bool wide = chunks > 1;
-    if (D <= 32) launch_gla<S, 1>(p, chunks, num_reqs, wide, stream);
-    else if (D <= 64) launch_gla<S, 2>(p, chunks, num_reqs, wide, stream);
-    else if (D <= 128) launch_gla<S, 4>(p, chunks, num_reqs, wide, stream);
-    else launch_gla<S, 8>(p, chunks, num_reqs, wide, stream);
+    if (D <= 32) pick_gla<S, 1>(p, chunks, num_reqs, wide, stream);
+    else if (D <= 64) pick_gla<S, 2>(p, chunks, num_reqs, wide, stream);
+    else if (D <= 128) pick_gla<S, 4>(p, chunks, num_reqs, wide, stream);
+    else pick_gla<S, 8>(p, chunks, num_reqs, wide, stream);
   });
   return launch_status();
 }

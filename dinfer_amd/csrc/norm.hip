@@ -834,3 +834,121 @@ extern "C" int dinfer_joined_norms(int dtype, const void* x, int64_t ld_x, int b
   });
   return launch_status();
 }
+
+// ---- a branch normed on its way into the stream -----------------------------------------------------------------
+//   stream[r] += (branch[r] - mean) / sqrt(var + eps) * w + b        (with a branch; var the mean of the squared deviations)
+//   out[r]     = stream[r]                                           (with an out: the stream in out's storage type)
+// for blocks whose sublayers read the stream itself and whose norms act on what the sublayers give.
+namespace {
+
+__global__ void __launch_bounds__(256) layernorm_add_kernel(const void* __restrict__ branch, int b_dt, int64_t ld_b,
+                                                            const float* __restrict__ w, const float* __restrict__ bias,
+                                                            float eps, void* __restrict__ stream, int s_dt, int64_t ld_s,
+                                                            void* __restrict__ out, int o_dt, int64_t width) {
+  extern __shared__ float row[];
+  __shared__ float red[16];
+  const int64_t r = blockIdx.x;
+  float mean = 0.f, inv = 0.f;
+  if (branch) {
+    float sum = 0.f, ss = 0.f;
+    for (int64_t i = threadIdx.x; i < width; i += blockDim.x) {
+      row[i] = ld_any(branch, r * ld_b + i, b_dt);
+      sum += row[i];
+    }
+    mean = block_sum(sum, red) / (float)width;
+    for (int64_t i = threadIdx.x; i < width; i += blockDim.x) ss = add_square(ss, row[i] - mean);   // (what it wrote itself)
+    inv = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+  }
+  for (int64_t i = threadIdx.x; i < width; i += blockDim.x) {
+    float x = ld_any(stream, r * ld_s + i, s_dt);
+    if (branch) {
+      x = round_any(x + ((row[i] - mean) * inv * w[i] + (bias ? bias[i] : 0.f)), s_dt);
+      st_any(stream, r * ld_s + i, s_dt, x);
+    }
+    if (out) st_any(out, r * width + i, o_dt, x);
+  }
+}
+
+// The same for a float stream and widths that are multiples of 8 up to 256 * 8 * ITERS: rows in registers, 16 or 32 bytes
+// at a time, the stream and the gains asked for with the branch.
+template <class S, int ITERS>
+__global__ void __launch_bounds__(256) layernorm_add_regs_kernel(const S* __restrict__ branch, int64_t ld_b,
+                                                                 const float* __restrict__ w, const float* __restrict__ bias,
+                                                                 float eps, float* __restrict__ stream, int64_t ld_s,
+                                                                 S* __restrict__ out, int64_t width) {
+  __shared__ float red[16];
+  const int64_t r = blockIdx.x;
+  const int n8 = (int)(width / 8);
+  float v[ITERS][8], x[ITERS][8], g[ITERS][8];
+  float sum = 0.f, ss = 0.f;
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int i = it * 256 + threadIdx.x;
+    if (i < n8) {
+      load8(branch + r * ld_b + (int64_t)i * 8, v[it]);
+      load8(stream + r * ld_s + (int64_t)i * 8, x[it]);
+      load8(w + (int64_t)i * 8, g[it]);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) sum += v[it][j];
+    }
+  }
+  const float mean = block_sum(sum, red) / (float)width;
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int i = it * 256 + threadIdx.x;
+    if (i < n8) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss = add_square(ss, v[it][j] - mean);
+    }
+  }
+  const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+#pragma unroll
+  for (int it = 0; it < ITERS; ++it) {
+    const int i = it * 256 + threadIdx.x;
+    if (i < n8) {
+      float b[8];
+      if (bias) load8(bias + (int64_t)i * 8, b);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[it][j] += (v[it][j] - mean) * inv * g[it][j] + (bias ? b[j] : 0.f);
+      store8(stream + r * ld_s + (int64_t)i * 8, x[it]);
+      if (out) store8(out + r * width + (int64_t)i * 8, x[it]);
+    }
+  }
+}
+
+template <class S>
+void launch_add_regs(const void* branch, int64_t ld_b, const float* w, const float* bias, float eps, void* stream_, int64_t ld_s,
+                     void* out, int64_t n_rows, int64_t width, hipStream_t stream) {
+#define LA(IT)                                                                                                          \
+  layernorm_add_regs_kernel<S, IT><<<(unsigned)n_rows, 256, 0, stream>>>((const S*)branch, ld_b, w, bias, eps, (float*)stream_, \
+                                                                         ld_s, (S*)out, width)
+  if (width <= 256 * 8) LA(1);
+  else if (width <= 256 * 8 * 2) LA(2);
+  else LA(4);
+#undef LA
+}
+
+}  // namespace
+
+// branch (may be null) [*, ld_b]; stream [*, ld_s], updated in place where a branch is given; out (may be null) dense
+// [n_rows, width]; w and bias (bias may be null) float. Width up to 16,384.
+extern "C" int dinfer_layernorm_add(const void* branch, int branch_dtype, int64_t ld_b, const float* w, const float* bias,
+                                    float eps, void* stream_, int stream_dtype, int64_t ld_s, void* out, int out_dtype,
+                                    int64_t n_rows, int64_t width, hipStream_t stream) {
+  if (n_rows <= 0) return OK;
+  if (width <= 0 || !stream_ || ld_s < width || (branch && (ld_b < width || !w)) || (!branch && !out) || n_rows > 0x7fffffff)
+    return ERR_BAD_SHAPE;
+  for (int dt : {branch_dtype, stream_dtype, out_dtype})
+    if (dt != DT_F32 && dt != DT_BF16) return ERR_BAD_DTYPE;
+  if (branch && stream_dtype == DT_F32 && (!out || out_dtype == branch_dtype) && width % 8 == 0 && width <= 256 * 8 * 4 &&
+      ld_s % 4 == 0 && ld_b % 8 == 0 && aligned16(stream_) && aligned16(branch) && aligned16(w) && aligned16(bias) &&
+      aligned16(out)) {
+    if (branch_dtype == DT_BF16) launch_add_regs<bf16>(branch, ld_b, w, bias, eps, stream_, ld_s, out, n_rows, width, stream);
+    else launch_add_regs<float>(branch, ld_b, w, bias, eps, stream_, ld_s, out, n_rows, width, stream);
+    return launch_status();
+  }
+  if (width > 16384) return ERR_UNSUPPORTED;
+  layernorm_add_kernel<<<(unsigned)n_rows, 256, (size_t)width * sizeof(float), stream>>>(
+      branch, branch_dtype, ld_b, w, bias, eps, stream_, stream_dtype, ld_s, out, out_dtype, width);
+  return launch_status();
+}

@@ -667,7 +667,7 @@ __global__ void __launch_bounds__(1024) qkv_row_post_vec_kernel(
 }  // namespace
 
 // qkv_post with norms over the whole projection: q_gain [heads head_dim], k_gain [kv_heads head_dim], float. Everything
-// else as there.
+// else as there. kv_heads 0: queries alone (a layer that reads another one's keys); nothing is written to the cache.
 extern "C" int dinfer_qkv_row_post(int dtype, void* qkv, int64_t tokens, int64_t ld, int64_t q_off, int64_t k_off,
                                    int64_t v_off, const float* q_gain, const float* k_gain, float eps,
                                    const int32_t* positions, const float* cos_sin, int rotary_dim, int style, void* k_cache,
@@ -676,7 +676,8 @@ extern "C" int dinfer_qkv_row_post(int dtype, void* qkv, int64_t tokens, int64_t
                                    int64_t ld_v_first, float v_share, hipStream_t stream) {
   if (v_dim <= 0) v_dim = head_dim;
   if (tokens <= 0) return OK;
-  if (heads <= 0 || kv_heads <= 0 || head_dim <= 0 || page_size <= 0 || tokens > 0x7fffffff || !q_gain || !k_gain)
+  if (heads <= 0 || kv_heads < 0 || head_dim <= 0 || page_size <= 0 || tokens > 0x7fffffff || !q_gain ||
+      (kv_heads > 0 && !k_gain) || (kv_heads == 0 && slot_mapping))
     return ERR_BAD_SHAPE;
   if (cos_sin && (rotary_dim <= 0 || rotary_dim > head_dim || rotary_dim % 2 != 0)) return ERR_BAD_SHAPE;
   if (style != 0 && style != 1) return ERR_UNSUPPORTED;

@@ -32,8 +32,8 @@ SIGNATURES = {
     "dinfer_latent_mfma_supports": ("latent", [_I, _I, _I]),
     "dinfer_latent_attn_mfma": ("latent", [_P, _L, _P, _L, _P, _L, _P, _P, _P, _L, _P, _P, _I, _L, _F, _I, _I, _I, _I, _I, _I, _P]),
     "dinfer_latent_attn_ref": ("latent", [_I, _P, _L, _P, _L, _P, _P, _L, _P, _P, _I, _L, _F, _I, _I, _I, _I, _I, _P]),
-    "dinfer_heads_nt": ("grouped", [_I, _P, _L, _L, _P, _L, _L, _P, _L, _L, _L, _L, _L, _L, _P, _L, _P]),
-    "dinfer_experts_nt": ("grouped", [_I, _I, _P, _L, _P, _L, _L, _P, _L, _L, _L, _P, _L, _I, _P, _P, _I, _I, _P, _P]),
+    "dinfer_heads_nt": ("grouped", [_I, _P, _L, _L, _P, _L, _L, _P, _L, _L, _L, _L, _L, _L, _P, _L, _I, _P]),
+    "dinfer_experts_nt": ("grouped", [_I, _I, _P, _L, _P, _L, _L, _P, _L, _L, _L, _P, _L, _I, _P, _P, _I, _I, _P, _F, _F, _P]),
     "dinfer_moe_tile_rows": ("grouped", [_I, _L, _I, _L, _L]),
     "dinfer_moe_route": ("grouped", [_I, _P, _L, _L, _P, _P, _I, _I, _I, _P, _P, _P, _P, _I, _P, _P]),
     "dinfer_moe_scatter": ("grouped", [_P, _L, _I, _I, _P, _P, _P, _L, _I, _P]),
@@ -49,6 +49,7 @@ SIGNATURES = {
         [_I, _P, _L, _L, _L, _L, _L, _P, _P, _F, _P, _P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _P, _L, _F, _P],
     ),
     "dinfer_group_rmsnorm": ("norm", [_P, _I, _L, _P, _I, _L, _P, _P, _P, _I, _F, _L, _L, _I, _P]),
+    "dinfer_layernorm_add": ("norm", [_P, _I, _L, _P, _P, _F, _P, _I, _L, _P, _I, _L, _L, _P]),
     "dinfer_joined_norms": ("norm", [_I, _P, _L, _I, _L, _P, _P, _P, _F, _P, _L, _P, _P, _F, _L, _L, _I, _P]),
     "dinfer_min_gru_chunk": ("scan", []),
     "dinfer_min_gru": ("scan", [_I, _P, _L, _L, _L, _L, _P, _P, _P, _P, _L, _P, _P, _P, _P, _L, _I, _L, _L, _L, _P]),
@@ -57,7 +58,7 @@ SIGNATURES = {
     "dinfer_channel_decay": ("linear_attention", [_I, _P, _L, _L, _I, _P, _P, _F, _P, _L, _L, _L, _P]),
     "dinfer_gla_recurrence": (
         "linear_attention",
-        [_I, _P, _P, _P, _L, _P, _L, _F, _P, _P, _P, _L, _P, _P, _P, _P, _L, _I, _L, _L, _I, _I, _I, _I, _P],
+        [_I, _P, _P, _P, _L, _P, _L, _F, _P, _P, _P, _L, _P, _P, _P, _P, _L, _I, _L, _L, _I, _I, _I, _I, _P, _I, _P],
     ),
     "dinfer_attn_paged_ref": (
         "attention_ref",
@@ -65,7 +66,7 @@ SIGNATURES = {
     ),
     "dinfer_attn_paged_ext": (
         "attention_ref",
-        [_I, _P, _L, _P, _L, _P, _P, _P, _L, _P, _P, _I, _L, _F, _I, _I, _P, _F, _I, _I, _I, _I, _I, _F, _P, _P],
+        [_I, _P, _L, _P, _L, _P, _P, _P, _L, _P, _P, _I, _L, _F, _I, _I, _P, _F, _I, _I, _I, _I, _I, _F, _P, _F, _I, _P],
     ),
     "dinfer_attn_paged_diff": (
         "attention_ref",
@@ -90,7 +91,7 @@ SIGNATURES = {
     "dinfer_decay_recurrence": ("decay", [_P, _L, _P, _L, _P, _L, _P, _L, _P, _L, _P, _P, _P, _P, _P, _L, _I, _I, _I, _I,
                                           _I, _P]),
     "dinfer_gated_group_norm": ("decay", [_I, _P, _L, _P, _L, _P, _I, _P, _L, _L, _P, _P, _L, _L, _L, _I, _I, _F, _F, _I,
-                                          _P]),
+                                          _I, _P]),
     "dinfer_streams_expand": ("streams", [_I, _P, _L, _P, _L, _L, _I, _I, _P]),
     "dinfer_streams_step": ("streams", [_I, _P, _L, _I, _I, _P, _P, _L, _P, _P, _P, _P, _P, _F, _P, _L, _P, _L, _L, _P]),
     "dinfer_attn_mfma_supports": ("attention", [_I, _I, _I, _I]),
@@ -101,7 +102,7 @@ SIGNATURES = {
     "dinfer_attn_flash_ext_supports": ("attention_ext", [_I, _I, _I, _I, _I, _I]),
     "dinfer_attn_flash_ext": (
         "attention_ext",
-        [_P, _L, _P, _L, _P, _P, _P, _L, _P, _P, _I, _I, _F, _I, _I, _P, _F, _F, _I, _I, _I, _I, _I, _P, _P],
+        [_P, _L, _P, _L, _P, _P, _P, _L, _P, _P, _I, _I, _F, _I, _I, _P, _F, _F, _I, _I, _I, _I, _I, _P, _F, _I, _P],
     ),
     "dinfer_attn_decode": (
         "attention",

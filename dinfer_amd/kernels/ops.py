@@ -223,6 +223,25 @@ def layernorm(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None, 
     return out
 
 
+def layernorm_add(stream: torch.Tensor, n_rows: int, *, branch: torch.Tensor | None = None, weight: torch.Tensor | None = None,
+                  bias: torch.Tensor | None = None, eps: float = 0.0, out: torch.Tensor | None = None) -> torch.Tensor | None:
+    """With a branch: stream += layernorm(branch) * weight + bias, in place (weight, bias float32). With an out:
+    out = stream, in out's type. Stream, branch and out may each be float32 or bfloat16."""
+    _need_gpu(stream, branch, weight, bias, out)
+    width = stream.shape[1]
+    assert stream.shape[0] >= n_rows and (branch is not None or out is not None)
+    if branch is not None:
+        assert branch.shape[1] == width and branch.shape[0] >= n_rows and weight is not None
+        assert all(t is None or (t.dtype == torch.float32 and t.numel() == width and t.is_contiguous()) for t in (weight, bias))
+    if out is not None:
+        assert out.is_contiguous() and out.shape[1] == width and out.shape[0] >= n_rows
+    lib.call("dinfer_layernorm_add", _ptr(branch), dtype_code(branch.dtype) if branch is not None else 0,
+             _rows(branch) if branch is not None else 0, _ptr(weight), _ptr(bias), float(eps), stream.data_ptr(),
+             dtype_code(stream.dtype), _rows(stream), _ptr(out), dtype_code(out.dtype) if out is not None else 0, n_rows, width,
+             _stream())
+    return out
+
+
 def rmsnorm_stream(stream: torch.Tensor, n_rows: int, *, branch: torch.Tensor | None = None,
                    branch_weight: torch.Tensor | None = None, branch_eps: float = 0.0, branch_offset: float = 0.0,
                    mult: float = 1.0, out: torch.Tensor | None = None, weight: torch.Tensor | None = None,
@@ -521,12 +540,13 @@ def decay_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: t
 def gated_group_norm(y: torch.Tensor, z: torch.Tensor, z_off: int, out: torch.Tensor, tokens: int, *, groups: int,
                      group: int, eps: float, weight: torch.Tensor | None = None, x: torch.Tensor | None = None,
                      skip: torch.Tensor | None = None, vdim: int = 0, col_off: int = 0, out_scale: float = 1.0,
-                     gate_first: bool = True) -> torch.Tensor:
+                     gate_first: bool = True, gate: str = "silu") -> torch.Tensor:
     """u = (y + skip[c // vdim] x) * silu(z[:, z_off + c]); out[:, col_off + c] = u / rms over c's group of `group`
     columns (eps inside the root) * weight[c] * out_scale. gate_first False: the gate multiplies after the norm
-    instead. y, x float32; z and out in the activations' type."""
+    instead. gate: "silu" or "sigmoid". y, x float32; z and out in the activations' type."""
     _need_gpu(y, z, out, weight, x, skip)
     n = groups * group
+    assert gate in ("silu", "sigmoid")
     assert y.dtype == torch.float32 and y.shape[1] >= n and z.dtype == out.dtype
     assert min(y.shape[0], z.shape[0], out.shape[0]) >= tokens and z_off + n <= z.shape[1] and col_off + n <= out.shape[1]
     assert weight is None or (weight.dtype == torch.float32 and weight.numel() == n and weight.is_contiguous())
@@ -535,7 +555,8 @@ def gated_group_norm(y: torch.Tensor, z: torch.Tensor, z_off: int, out: torch.Te
         assert skip.dtype == torch.float32 and vdim > 0 and skip.numel() * vdim == n
     lib.call("dinfer_gated_group_norm", dtype_code(out.dtype), y.data_ptr(), _rows(y), _ptr(x) if skip is not None else None,
              _rows(x) if skip is not None else 0, _ptr(skip), int(vdim), z.data_ptr(), _rows(z), z_off, _ptr(weight),
-             out.data_ptr(), _rows(out), col_off, tokens, groups, group, float(eps), float(out_scale), 1 if gate_first else 0, _stream())
+             out.data_ptr(), _rows(out), col_off, tokens, groups, group, float(eps), float(out_scale), 1 if gate_first else 0,
+             1 if gate == "sigmoid" else 0, _stream())
     return out
 
 
@@ -567,29 +588,35 @@ def gla_cuts(tokens: int, max_rows: int, num_reqs: int, heads: int, vdim: int) -
     return bool(lib.get("dinfer_gla_cuts")(tokens, max_rows, num_reqs, heads, vdim))
 
 
-def gla_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, state: torch.Tensor,
+def gla_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor | None, state: torch.Tensor,
                    out: torch.Tensor, *, q_scale: float, notes: torch.Tensor | None, products: torch.Tensor | None,
                    state_slots: torch.Tensor, cu_seqlens: torch.Tensor, seq_lens: torch.Tensor, num_reqs: int, tokens: int,
-                   max_rows: int, cut: bool, heads: int, dim: int, vdim: int) -> torch.Tensor:
+                   max_rows: int, cut: bool, heads: int, dim: int, vdim: int, fixed: torch.Tensor | None = None,
+                   act: bool = False) -> torch.Tensor:
     """Per request and head, token by token: S <- diag(decay) S + k v^T, out = S^T (q * q_scale). q, k [T, heads dim] and v
     [T, heads vdim] are column blocks of one buffer as the projections left them; decay float32 [T, heads dim]. state
     [slots, heads, vdim, dim] float32, updated in place; out [T, heads vdim] float32. cut: in chunks side by side, with
-    scratch notes [places, heads, vdim, dim] and products [places, heads, dim] (gla_places of the step at least)."""
-    _need_gpu(q, k, v, decay, state, out, notes, products, state_slots, cu_seqlens, seq_lens)
+    scratch notes [places, heads, vdim, dim] and products [places, heads, dim] (gla_places of the step at least).
+    fixed (float32 [heads], in place of decay): one constant decay a head. act: q, k and v are the silu of the operands."""
+    assert (decay is None) != (fixed is None) and (fixed is not None or not act)
+    if fixed is not None:
+        assert fixed.dtype == torch.float32 and fixed.numel() == heads and fixed.is_contiguous()
+    _need_gpu(q, k, v, decay, fixed, state, out, notes, products, state_slots, cu_seqlens, seq_lens)
     assert q.dtype == k.dtype == v.dtype and _rows(q) == _rows(k) == _rows(v)
-    assert decay.dtype == state.dtype == out.dtype == torch.float32 and state.is_contiguous()
-    assert tuple(state.shape[1:]) == (heads, vdim, dim) and out.shape[1] >= heads * vdim and decay.shape[1] >= heads * dim
+    assert state.dtype == out.dtype == torch.float32 and state.is_contiguous()
+    assert decay is None or (decay.dtype == torch.float32 and decay.shape[1] >= heads * dim and decay.shape[0] >= tokens)
+    assert tuple(state.shape[1:]) == (heads, vdim, dim) and out.shape[1] >= heads * vdim
     assert q.shape[1] >= heads * dim and k.shape[1] >= heads * dim and v.shape[1] >= heads * vdim
-    assert min(t.shape[0] for t in (q, k, v, decay, out)) >= tokens
+    assert min(t.shape[0] for t in (q, k, v, out)) >= tokens
     places = 0
     if cut:
         assert notes is not None and notes.dtype == products.dtype == torch.float32
         assert notes.is_contiguous() and products.is_contiguous()
         places = min(notes.numel() // (heads * vdim * dim), products.numel() // (heads * dim))
     lib.call("dinfer_gla_recurrence", dtype_code(q.dtype), q.data_ptr(), k.data_ptr(), v.data_ptr(), _rows(q),
-             decay.data_ptr(), _rows(decay), float(q_scale), state.data_ptr(), _ptr(notes) if cut else 0,
+             _ptr(decay), _rows(decay) if decay is not None else 0, float(q_scale), state.data_ptr(), _ptr(notes) if cut else 0,
              _ptr(products) if cut else 0, places, state_slots.data_ptr(), cu_seqlens.data_ptr(), seq_lens.data_ptr(),
-             out.data_ptr(), _rows(out), num_reqs, tokens, max_rows, int(cut), heads, dim, vdim, _stream())
+             out.data_ptr(), _rows(out), num_reqs, tokens, max_rows, int(cut), heads, dim, vdim, _ptr(fixed), int(act), _stream())
     return out
 
 
@@ -761,9 +788,10 @@ def latent_attn_mfma(qa: torch.Tensor, out: torch.Tensor, cache: torch.Tensor, c
 
 # ---- many small products in one launch ---------------------------------------------------------------
 def heads_nt(a: torch.Tensor, a_off: int, a_stride: int, w: torch.Tensor, out: torch.Tensor, c_off: int, c_stride: int,
-             m: int, *, gate: torch.Tensor | None = None, gate_off: int = 0) -> torch.Tensor:
+             m: int, *, gate: torch.Tensor | None = None, gate_off: int = 0, gate_entries: bool = False) -> torch.Tensor:
     """For every head z: out[:m, c_off + z*c_stride : ... + N] = a[:m, a_off + z*a_stride : ... + K] @ w[z].T with
-    w [heads, N, K]; gate: the rows of head z are multiplied by sigmoid(gate[:, gate_off + z])."""
+    w [heads, N, K]; gate: the rows of head z are multiplied by sigmoid(gate[:, gate_off + z]), with gate_entries entry n of
+    them by sigmoid(gate[:, gate_off + z*N + n])."""
     _need_gpu(a, w, out, gate)
     heads, n, k = w.shape
     assert w.is_contiguous() and a.dtype == w.dtype == out.dtype
@@ -771,10 +799,10 @@ def heads_nt(a: torch.Tensor, a_off: int, a_stride: int, w: torch.Tensor, out: t
     assert a_off + (heads - 1) * a_stride + k <= a.shape[1] and c_off + (heads - 1) * c_stride + n <= out.shape[1]
     es = a.element_size()
     if gate is not None:
-        assert gate.dtype == a.dtype and gate.shape[0] >= m and gate_off + heads <= gate.shape[1]
+        assert gate.dtype == a.dtype and gate.shape[0] >= m and gate_off + heads * (n if gate_entries else 1) <= gate.shape[1]
     lib.call("dinfer_heads_nt", dtype_code(a.dtype), a.data_ptr() + a_off * es, _rows(a), a_stride, w.data_ptr(), k, n * k,
              out.data_ptr() + c_off * es, _rows(out), c_stride, m, n, k, heads,
-             gate.data_ptr() + gate_off * es if gate is not None else 0, _rows(gate) if gate is not None else 0, _stream())
+             gate.data_ptr() + gate_off * es if gate is not None else 0, _rows(gate) if gate is not None else 0, int(gate_entries), _stream())
     return out
 
 
@@ -837,12 +865,15 @@ def moe_scatter(idx: torch.Tensor, entries: int, experts: int, offsets: torch.Te
 
 def experts_nt(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, entries: int, tiles: torch.Tensor,
                offsets: torch.Tensor, perm: torch.Tensor, *, gated: bool, a_div: int, c_to_perm: bool,
-               tile_rows: int, act: str | None = None, row_scale: torch.Tensor | None = None) -> torch.Tensor:
+               tile_rows: int, act: str | None = None, row_scale: torch.Tensor | None = None,
+               clamp: tuple | None = None) -> torch.Tensor:
     """The products of all experts in one launch. w [experts, rows, K]; gated: rows = 2 N, gate rows first, and
     out = silu(a Wg^T) * (a Wu^T). a_div > 0: the row of sorted place i is a[perm[i] // a_div] (the step's tokens),
     0: a[i]. c_to_perm: the result of sorted place i goes to out[perm[i]], else to out[i]. tile_rows: what moe_scatter
     made the work list with. act (not gated): "silu", "gelu" (error function) or "relu2" on every result. row_scale: float32,
-    a factor an entry that multiplies the entry's row of a (on the float sums, before the activation)."""
+    a factor an entry that multiplies the entry's row of a (on the float sums, before the activation). clamp (limit, slope),
+    gated: out = g sigmoid(slope g) (u + 1) from g = min(a Wg^T, limit) and u = a Wu^T clamped to [-limit, limit]."""
+    assert clamp is None or (gated and clamp[0] > 0)
     _need_gpu(a, w, out, tiles, offsets, perm, row_scale)
     assert row_scale is None or (row_scale.dtype == torch.float32 and row_scale.is_contiguous() and row_scale.numel() >= entries)
     if act is not None and (gated or act not in EXPERT_ACTS):
@@ -853,7 +884,8 @@ def experts_nt(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, entries: int
     assert out.shape[0] >= entries and (a_div > 0 or a.shape[0] >= entries)
     lib.call("dinfer_experts_nt", dtype_code(a.dtype), 1 if gated else EXPERT_ACTS[act] if act else 0, a.data_ptr(), _rows(a), w.data_ptr(), k,
              rows * k, out.data_ptr(), _rows(out), n, k, tiles.data_ptr(), moe_max_tiles(entries, experts, tile_rows),
-             int(tile_rows), offsets.data_ptr(), perm.data_ptr(), int(a_div), 1 if c_to_perm else 0, _ptr(row_scale), _stream())
+             int(tile_rows), offsets.data_ptr(), perm.data_ptr(), int(a_div), 1 if c_to_perm else 0, _ptr(row_scale),
+             float(clamp[0]) if clamp else 0.0, float(clamp[1]) if clamp else 0.0, _stream())
     return out
 
 
@@ -927,7 +959,7 @@ def qkv_post(qkv: torch.Tensor, tokens: int, *, heads: int, kv_heads: int, head_
     multiplied by 1 + coef ln(floor((p + 1) / every) + 1) at position p, together with the norm. q_head_scale: float32
     [heads], q of head h is multiplied by its entry with the norm (a temperature on the head's scores).
     whole: the norms run over the whole projection, all heads of a token at once (gains float32 [heads * head_dim] and
-    [kv_heads * head_dim]). v_first [T, kv_heads * v_dim]: the cached values are (1 - v_share) v + v_share v_first.
+    [kv_heads * head_dim]); with kv_heads 0 there are queries alone (nothing is cached). v_first [T, kv_heads * v_dim]: the cached values are (1 - v_share) v + v_share v_first.
     v_dim: the size of a value head where it is not head_dim. v_cache None beside a k_cache: the values are not stored
     (a layer whose values are its keys reads them from the key pages).
 
@@ -947,8 +979,9 @@ def qkv_post(qkv: torch.Tensor, tokens: int, *, heads: int, kv_heads: int, head_
     first = (_ptr(v_first), _rows(v_first) if v_first is not None else 0, float(v_share))
     if whole:
         assert q_temp is None and q_head_scale is None and gain_offset == 0.0
-        assert q_gain.dtype == k_gain.dtype == torch.float32 and q_gain.is_contiguous() and k_gain.is_contiguous()
-        assert q_gain.numel() == heads * head_dim and k_gain.numel() == kv_heads * head_dim
+        assert q_gain.dtype == torch.float32 and q_gain.is_contiguous() and q_gain.numel() == heads * head_dim
+        assert k_gain is None if kv_heads == 0 else (k_gain.dtype == torch.float32 and k_gain.is_contiguous()
+                                                     and k_gain.numel() == kv_heads * head_dim)
     elif q_gain is not None:
         assert q_gain.numel() == head_dim and k_gain is not None and k_gain.numel() == head_dim
         wf32 = _is_param_f32(q_gain, qkv.dtype)
@@ -969,7 +1002,7 @@ def qkv_post(qkv: torch.Tensor, tokens: int, *, heads: int, kv_heads: int, head_
         assert k_cache.dtype == qkv.dtype and (v_cache is None or v_cache.dtype == qkv.dtype)
     if whole:
         lib.call("dinfer_qkv_row_post", dtype_code(qkv.dtype), qkv.data_ptr(), tokens, ld, q_off, k_off, v_off,
-                 q_gain.data_ptr(), k_gain.data_ptr(), float(eps), positions.data_ptr(), _ptr(cos_sin), rotary_dim,
+                 q_gain.data_ptr(), _ptr(k_gain), float(eps), positions.data_ptr(), _ptr(cos_sin), rotary_dim,
                  rope_style, _ptr(k_cache), _ptr(v_cache), _ptr(slot_mapping), heads, kv_heads, head_dim, page_size,
                  int(token_runs), vd, _ptr(bias), *first, _stream())
         return
@@ -984,12 +1017,13 @@ def attn_paged_ext(q: torch.Tensor, out: torch.Tensor, k_cache: torch.Tensor, v_
                    block_table: torch.Tensor, cu_seqlens: torch.Tensor, seq_lens: torch.Tensor, num_reqs: int,
                    tokens: int, *, scale: float, window: int, heads: int, kv_heads: int, head_dim: int, page_size: int,
                    v_dim: int | None = None, keep_first: int = 0, sinks: torch.Tensor | None = None,
-                   slope_exp: float = 0.0, out_scale: float = 1.0,
-                   sigmoid_bias: torch.Tensor | None = None) -> torch.Tensor:
+                   slope_exp: float = 0.0, out_scale: float = 1.0, sigmoid_bias: torch.Tensor | None = None,
+                   softcap: float = 0.0, chunk: int = 0) -> torch.Tensor:
     """The plain kernel with its options: keys j < keep_first stay visible behind the window; sinks (float32 [heads])
     join the softmax's denominator; slope_exp E takes 2^(-E (h + 1) / heads) * distance off the scores; values of size
     v_dim, or read from the key pages (v_cache None); the output times out_scale; sigmoid_bias (float32 [heads]): the
-    weights are sigmoid(score + bias), not normalised. Any storage type."""
+    weights are sigmoid(score + bias), not normalised; softcap C: the scores are C tanh(score / C), before the distance
+    bias; chunk N: a row sees the keys of its own chunk of N positions only. Any storage type."""
     _need_gpu(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, sinks, sigmoid_bias)
     if sigmoid_bias is not None:
         assert sinks is None and sigmoid_bias.dtype == torch.float32 and sigmoid_bias.numel() == heads
@@ -1004,7 +1038,8 @@ def attn_paged_ext(q: torch.Tensor, out: torch.Tensor, k_cache: torch.Tensor, v_
     lib.call("dinfer_attn_paged_ext", dtype_code(q.dtype), q.data_ptr(), _rows(q), out.data_ptr(), _rows(out),
              k_cache.data_ptr(), _ptr(v_cache), block_table.data_ptr(), block_table.shape[1], cu_seqlens.data_ptr(),
              seq_lens.data_ptr(), num_reqs, tokens, float(scale), int(window), int(keep_first), _ptr(sinks),
-             float(slope_exp), heads, kv_heads, head_dim, vd, page_size, float(out_scale), _ptr(sigmoid_bias), _stream())
+             float(slope_exp), heads, kv_heads, head_dim, vd, page_size, float(out_scale), _ptr(sigmoid_bias),
+             float(softcap), int(chunk), _stream())
     return out
 
 
@@ -1098,8 +1133,8 @@ def attn_flash(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, num_
 def attn_flash_ext(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, num_reqs: int, max_q_len: int, *,
                    scale: float, window: int, heads: int, kv_heads: int, head_dim: int, page_size: int,
                    keep_first: int = 0, sinks: torch.Tensor | None = None, slope_exp: float = 0.0,
-                   out_scale: float = 1.0, v_dim: int | None = None,
-                   sigmoid_bias: torch.Tensor | None = None) -> torch.Tensor:
+                   out_scale: float = 1.0, v_dim: int | None = None, sigmoid_bias: torch.Tensor | None = None,
+                   softcap: float = 0.0, chunk: int = 0) -> torch.Tensor:
     """The matrix-core flash kernel with the options of attn_paged_ext (bfloat16, sizes attn_flash_ext_supports names,
     values in value pages), for prompt portions and single rows alike."""
     _need_gpu(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, sinks, sigmoid_bias)
@@ -1112,7 +1147,8 @@ def attn_flash_ext(q, out, k_cache, v_cache, block_table, cu_seqlens, seq_lens, 
     lib.call("dinfer_attn_flash_ext", q.data_ptr(), _rows(q), out.data_ptr(), _rows(out), k_cache.data_ptr(),
              v_cache.data_ptr(), block_table.data_ptr(), block_table.shape[1], cu_seqlens.data_ptr(), seq_lens.data_ptr(),
              num_reqs, max_q_len, float(scale), int(window), int(keep_first), _ptr(sinks), float(slope_exp),
-             float(out_scale), heads, kv_heads, head_dim, vd, page_size, _ptr(sigmoid_bias), _stream())
+             float(out_scale), heads, kv_heads, head_dim, vd, page_size, _ptr(sigmoid_bias), float(softcap), int(chunk),
+             _stream())
     return out
 
 

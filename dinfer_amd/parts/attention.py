@@ -20,8 +20,11 @@ of k over the whole projection, all heads of a token sharing one root mean squar
 size); weights that are sigmoids of the scores plus a learned bias a head, not normalised over the keys (`sigmoid_bias`, a
 tensor [heads]); a bias on the output projection (`out_bias`); values mixed with another layer's (`value_mix`, a tensor of
 one number, lambda): the layer with "keep" leaves its values of the step where they are until the step's end, a layer with
-"mix" caches (1 - lambda) v + lambda v_kept of the same token. A layer that uses any
-option runs the flash kernel with options on the matrix cores where its sizes allow, else the plain kernel with options
+"mix" caches (1 - lambda) v + lambda v_kept of the same token; scores softly capped, C tanh(s / C) (`softcap`); positions in
+chunks of `chunk` tokens, counted from a request's first one, a query seeing the keys of its own chunk only; no keys and
+values of the layer's own (`shares_cache`: it reads the cache of the run entry it is given, with queries, mask, scale and
+cap of its own); `cache_window`: how many keys back the cache must keep where that is more than the layer's own mask asks for (layers that
+read it may look further back; None: every key). A layer that uses any option runs the flash kernel with options on the matrix cores where its sizes allow, else the plain kernel with options
 (csrc/attention_ref.hip), for prompt portions and single rows alike; the matrix-core kernels serve the others.
 """
 from __future__ import annotations
@@ -54,7 +57,8 @@ class Attention(Mixer):
                  qk_unit_eps: float | None = None, q_temp: tuple | None = None, sink_value: float | None = None,
                  gate: str | None = None, gate_heads: bool = False, head_temp: bool = False,
                  qk_row_eps: float | None = None, sigmoid_bias: bool = False, out_bias: bool = False,
-                 value_mix: str | None = None):
+                 value_mix: str | None = None, softcap: float | None = None, chunk: int | None = None,
+                 shares_cache: bool = False, cache_window: int | None = -1):
         if heads % kv_heads:
             raise ValueError(f"heads {heads} not divisible by kv_heads {kv_heads}")
         if head_dim <= 0 or head_dim > ops.MAX_HEAD_DIM:   # said at build, not at the first step
@@ -98,14 +102,29 @@ class Attention(Mixer):
         if value_mix not in (None, "keep", "mix") or (value_mix and (self.bias or self.values_are_keys)):
             raise ValueError(f"attention: value_mix {value_mix!r} (known: 'keep', 'mix'; without biases and with values of "
                              "their own)")
+        self.softcap, self.chunk, self.shares_cache = float(softcap or 0.0), int(chunk or 0), bool(shares_cache)
+        if self.softcap < 0 or self.chunk < 0 or (self.softcap and self.sigmoid):
+            raise ValueError(f"attention: softcap {softcap} or chunk {chunk} out of range, or a cap under sigmoid weights")
+        if self.shares_cache and (self.bias or self.values_are_keys or value_mix or qk_norm is not None or qk_unit_eps is not None
+                                  or POSITION_ENCODINGS.get(position.kind) is not POSITION_ENCODINGS.get("none")):
+            raise ValueError("attention: a layer that reads another one's keys takes norms over the whole projection or none, and "
+                             "no biases, rotation, or values of another kind")
+        if self.chunk and self.keep_first and not window:
+            raise ValueError("attention: kept first keys beside chunks are not built")
+        # the keys the cache keeps: those of the window, or of a chunk as long as it may reach back
+        own = min((n for n in (window, self.chunk) if n), default=None)
+        self.cache_window = own if cache_window == -1 else cache_window
+        if self.cache_window is not None and (own is None or self.cache_window < own):
+            raise ValueError(f"attention: a cache of {self.cache_window} keys is less than the mask sees")
         # what the matrix-core kernels do not do runs through the plain kernel with options
         self.extended = bool(self.v_dim != head_dim or self.keep_first or self.sink or self.slope_exp
                              or self.values_are_keys or self.out_scale != 1.0 or self.bias or qk_unit_eps is not None
                              or self.q_temp is not None or self.sink_value is not None or gate is not None
                              or self.head_temp or self.qk_row_eps is not None or self.sigmoid or self.out_bias_on
-                             or value_mix is not None)
-        self.q_size, self.kv_size = heads * head_dim, kv_heads * head_dim
-        self.v_size = 0 if self.values_are_keys else kv_heads * self.v_dim
+                             or value_mix is not None or self.softcap or self.chunk or self.shares_cache)
+        self.q_size = heads * head_dim
+        self.kv_size = 0 if self.shares_cache else kv_heads * head_dim
+        self.v_size = 0 if self.values_are_keys or self.shares_cache else kv_heads * self.v_dim
         self.g_size = (heads if self.gate_heads else heads * self.v_dim) if gate is not None else 0
         self.temps = None
         self.g_off = self.q_size + self.kv_size + self.v_size
@@ -126,17 +145,18 @@ class Attention(Mixer):
 
     def cache_spec(self):
         # (asked after bind, which settles whether values that are the keys are stored a second time)
-        return KVSpec(self.kv_heads, self.head_dim, self.window, v_dim=self.v_dim, keep_first=self.keep_first,
+        return KVSpec(self.kv_heads, self.head_dim, self.cache_window, v_dim=self.v_dim, keep_first=self.keep_first,
                       values=self.stores_values)
 
     def tensors(self):
         D, Hd, nm = self.head_dim, self.hidden, self.names
         t = {
             nm["q"]: TensorSpec((self.q_size, Hd)),
-            nm["k"]: TensorSpec((self.kv_size, Hd)),
             nm["o"]: TensorSpec((Hd, self.heads * self.v_dim)),
         }
-        if not self.values_are_keys:
+        if not self.shares_cache:
+            t[nm["k"]] = TensorSpec((self.kv_size, Hd))
+        if self.v_size:
             t[nm["v"]] = TensorSpec((self.v_size, Hd))
         if self.q_norm is not None:
             for which, norm in (("q_norm", self.q_norm), ("k_norm", self.k_norm)):
@@ -154,7 +174,8 @@ class Attention(Mixer):
             t[nm["temp"]] = TensorSpec((self.heads,), init="gain")
         if self.qk_row_eps is not None:
             t[nm["q_norm"]] = TensorSpec((self.q_size,), init="gain")
-            t[nm["k_norm"]] = TensorSpec((self.kv_size,), init="gain")
+            if not self.shares_cache:
+                t[nm["k_norm"]] = TensorSpec((self.kv_size,), init="gain")
         if self.sigmoid:
             t[nm["sigmoid_bias"]] = TensorSpec((self.heads,), init="zeros")
         if self.out_bias_on:
@@ -177,8 +198,10 @@ class Attention(Mixer):
     def weight_rows(self, get) -> torch.Tensor:
         # q, k, v rows concatenated into one [(H + 2 Hkv) D, hidden] operand (model.rs:141-165)
         nm = self.names
-        rows = [get(nm["q"], compute=True), get(nm["k"], compute=True)]
-        if not self.values_are_keys:
+        rows = [get(nm["q"], compute=True)]
+        if not self.shares_cache:
+            rows.append(get(nm["k"], compute=True))
+        if self.v_size:
             rows.append(get(nm["v"], compute=True))
         if self.gate is not None:
             rows.append(get(nm["g"], compute=True))
@@ -212,7 +235,8 @@ class Attention(Mixer):
         if self.head_temp:
             self.temps = get(nm["temp"]).float().contiguous()
         if self.qk_row_eps is not None:
-            self.row_gains = tuple(get(nm[k]).float().contiguous() for k in ("q_norm", "k_norm"))
+            self.row_gains = tuple(None if k == "k_norm" and self.shares_cache else get(nm[k]).float().contiguous()
+                                   for k in ("q_norm", "k_norm"))
         if self.sigmoid:
             self.sigmoid_biases = get(nm["sigmoid_bias"]).float().contiguous()
         if self.value_mix == "mix":      # (the layer that keeps its values has the tensor too and does not use it)
@@ -309,6 +333,15 @@ class Attention(Mixer):
         eps = qn.eps if qn else (self.qk_unit_eps or 0.0)
         if self.row_gains is not None:
             (q_gain, k_gain), eps = self.row_gains, self.qk_row_eps
+        if self.shares_cache:
+            if self.row_gains is not None:      # the queries' norm is all there is to do before the scores
+                ops.qkv_post(qkv_buf, T, heads=self.heads, kv_heads=0, head_dim=self.head_dim, q_off=col, k_off=col, v_off=col,
+                             positions=batch.positions, page_size=self.page_size, q_gain=q_gain, k_gain=None, eps=eps,
+                             gain_offset=0.0, cos_sin=None, rotary_dim=0, rope_style=0, k_cache=None, v_cache=None,
+                             slot_mapping=None, whole=True)
+            self._attend_ext(qkv_buf, col, attn_buf, out_col, batch, cache)
+            self._gate(qkv_buf, col, attn_buf, out_col, T)
+            return
         ops.qkv_post(qkv_buf, T, heads=self.heads, kv_heads=self.kv_heads, head_dim=self.head_dim, q_off=col,
                      k_off=col + self.q_size,     # (values that are the keys: the key columns as the product left them)
                      v_off=col + self.q_size + (0 if self.values_are_keys else self.kv_size),
@@ -320,8 +353,11 @@ class Attention(Mixer):
                      q_head_scale=self.temps, whole=self.row_gains is not None, v_first=self.kept_values,
                      v_share=self.value_share)
         self._attend_ext(qkv_buf, col, attn_buf, out_col, batch, cache)
+        self._gate(qkv_buf, col, attn_buf, out_col, T)
+
+    def _gate(self, qkv_buf, col, attn_buf, out_col, T):
         if self.gate is not None:
-            n = self.heads * vd
+            vd, n = self.v_dim, self.heads * self.v_dim
             ops.gate(attn_buf[:, out_col:out_col + n], qkv_buf[:, col + self.g_off:col + self.g_off + self.g_size], T,
                      self.gate, group=vd if self.gate_heads else 1)
 
@@ -333,13 +369,14 @@ class Attention(Mixer):
                                window=self.window or 0, heads=self.heads, kv_heads=self.kv_heads, head_dim=self.head_dim,
                                page_size=self.page_size, keep_first=self.keep_first, sinks=self.sinks,
                                slope_exp=self.slope_exp, out_scale=self.out_scale, v_dim=vd,
-                               sigmoid_bias=self.sigmoid_biases)
+                               sigmoid_bias=self.sigmoid_biases, softcap=self.softcap, chunk=self.chunk)
             return
         ops.attn_paged_ext(qkv_buf[:, col:], attn_buf[:, out_col:], cache.k, cache.v, batch.block_table[g],
                            batch.cu_seqlens, batch.seq_lens, batch.num_reqs, T, scale=self.scale,
                            window=self.window or 0, heads=self.heads, kv_heads=self.kv_heads, head_dim=self.head_dim,
                            page_size=self.page_size, v_dim=vd, keep_first=self.keep_first, sinks=self.sinks,
-                           slope_exp=self.slope_exp, out_scale=self.out_scale, sigmoid_bias=self.sigmoid_biases)
+                           slope_exp=self.slope_exp, out_scale=self.out_scale, sigmoid_bias=self.sigmoid_biases,
+                           softcap=self.softcap, chunk=self.chunk)
 
     def _project_out(self, T, into):
         if into is not None and self.o_bias is None:

@@ -220,6 +220,93 @@ class SandwichBlock(Block):
         return Carried(None, None, 0, 0.0, self.hidden, next_norm, hidden, self.normed, T, ready=True)
 
 
+class NormedBranch:
+    """A sublayer's output that is still to be normed and added to the stream, left pending by an `outnorm` block so that
+    the kernel which makes the next reader's copy of the stream does it in the same pass. `settle(rows)` does it alone."""
+    __slots__ = ("stream", "branch", "norm")
+
+    def __init__(self, stream, branch, norm):
+        self.stream, self.branch, self.norm = stream, branch, norm
+
+    def settle(self, rows: int, out=None) -> None:
+        ops.layernorm_add(self.stream, rows, branch=self.branch, weight=self.norm.weight, bias=self.norm.bias, eps=self.norm.eps,
+                          out=out)
+
+
+@BLOCKS.register("outnorm")
+class OutNormBlock(Block):
+    """Norms on the sublayers' outputs only; the sublayers read the stream itself:
+
+        h += norm_a(mixer(h));   h += norm_b(ff(h))
+
+    One kernel a sublayer boundary norms the branch, adds it to the stream and, where the stream is kept wider than the
+    engine's dtype, writes the copy in that dtype which the next sublayer's products read (else they read the stream).
+    The last sublayer's branch is left pending for the next block's first kernel. params: mixer_prefix, ff_prefix and the
+    norms' names; the norms must be layer norms (gain and optional bias)."""
+
+    def __init__(self, hidden: int, layer: LayerSpec, mixer_prefix: str = "mix.", ff_prefix: str = "mlp.",
+                 norm_a: str = "norm1", norm_b: str = "norm2"):
+        self.hidden = hidden
+        self.mixer = MIXERS.get(layer.mixer.kind)(hidden=hidden, **layer.mixer.params)
+        self.ff = FEED_FORWARDS.get(layer.feed_forward.kind)(hidden=hidden, **layer.feed_forward.params)
+        if getattr(self.ff, "absent", False):
+            self.ff = None
+        ncls = NORMS.get(layer.norm.kind)
+        self.norms = [(n, ncls(hidden, **layer.norm.params)) for n in ([norm_a] if self.ff is None else [norm_a, norm_b])]
+        if any(not hasattr(n, "has_bias") for _, n in self.norms):
+            raise ValueError("norms on the outputs alone: the arrangement takes layer norms (gain and optional bias)")
+        self.prefixes = (mixer_prefix, ff_prefix)
+
+    def _parts(self):
+        out = [(self.prefixes[0], self.mixer)] + list(self.norms)
+        if self.ff is not None:
+            out.append((self.prefixes[1], self.ff))
+        return out
+
+    @property
+    def capturable(self):
+        return all(part.capturable for _, part in self._parts())
+
+    @property
+    def capturable_portions(self):
+        return all(part.capturable and part.capturable_portions for _, part in self._parts())
+
+    def tensors(self):
+        return {p + n: s for p, part in self._parts() for n, s in part.tensors().items()}
+
+    def load(self, get):
+        for p, part in self._parts():
+            part.load(_sub(get, p))
+
+    def bind(self, ctx):
+        for _, part in self._parts():
+            part.bind(ctx)
+        self.copy = ctx.workspace.buffer("normed", self.hidden)
+
+    def _read(self, hidden, pending, T):
+        """Settles what is pending; returns what the next sublayer reads."""
+        same = hidden.dtype == self.copy.dtype
+        if isinstance(pending, NormedBranch):
+            pending.settle(T, None if same else self.copy)
+        else:
+            if isinstance(pending, torch.Tensor):      # a block of another kind left its last branch to be added
+                ops.add_rows(hidden, T, a=pending)
+            elif pending is not None and not isinstance(pending, Carried):     # (a Carried: the stream is complete)
+                raise TypeError(f"a block that reads the stream itself cannot follow a pending {type(pending).__name__}")
+            if not same:
+                ops.layernorm_add(hidden, T, out=self.copy)
+        return hidden if same else self.copy
+
+    def forward(self, hidden, pending, batch, cache: CacheView):
+        T = batch.num_tokens
+        a = self.mixer.forward(self._read(hidden, pending, T), batch, cache)
+        pending = NormedBranch(hidden, a, self.norms[0][1])
+        if self.ff is not None:
+            f = self.ff.forward(self._read(hidden, pending, T), batch)
+            pending = NormedBranch(hidden, f, self.norms[1][1])
+        return pending
+
+
 class StreamsWrite:
     """A sublayer's output that is still to be written into the residual streams (x_t <- sum_s mix[s, t] x_s +
     out[t] y): left pending by a `streams` block so that the kernel which reads the streams next does the write in the

@@ -8,7 +8,8 @@ latent size:
     c = rmsnorm(c') * w                              kr = rot(kr'),  qr_h <- rot(qr_h)
     kn_h = Wuk_h c,   v_h = Wuv_h c
     s_ij = scale * (qn_h,i . kn_h,j + qr_h,i . kr_j),   j <= i  (j > i - window where a window is given)
-    y = Wo concat_h( sigmoid(Wg h)_h * sum_j softmax(s)_ij v_h,j )        (the gate only with `gated`)
+    y = Wo concat_h( sigmoid(Wg h)_h * sum_j softmax(s)_ij v_h,j )        (the gate only with `gated`: one number a head;
+                                                                           gated="entries": one an entry of the heads)
 
 The cache holds [c | kr] per token (LatentSpec). The products with Wuk and Wuv are done on the query side:
 qa_h = Wuk_h^T qn_h, s = scale * <[qa_h | qr_h], [c | kr]>, and the attention's output in latent space is multiplied
@@ -38,7 +39,7 @@ class LatentAttention(Mixer):
     capturable_portions = True   # the choice of kernels follows the step's counts alone
 
     def __init__(self, hidden: int, heads: int, dim: int, rot_dim: int, vdim: int, rank: int, scale: float,
-                 position: PartSpec, latent_norm: PartSpec, gated: bool = True, shares_cache: bool = False,
+                 position: PartSpec, latent_norm: PartSpec, gated: bool | str = True, shares_cache: bool = False,
                  window: int | None = None,
                  names: tuple = ("q", "dkv", "dkv.norm", "uk", "uv", "g", "o"), q_rank: int | None = None,
                  q_names: tuple = ("dq", "dq.norm", "uq")):
@@ -46,7 +47,11 @@ class LatentAttention(Mixer):
             raise ValueError(f"latent attention: rank {rank} with rot_dim {rot_dim} has no kernel (rank up to "
                              f"{ops.LATENT_MAX_RANK}, rank + rot_dim up to {ops.LATENT_MAX_KEY})")
         self.hidden, self.heads, self.dim, self.rot_dim, self.vdim, self.rank = hidden, heads, dim, rot_dim, vdim, rank
-        self.scale, self.gated, self.shares_cache, self.window = float(scale), gated, shares_cache, window
+        if gated not in (True, False, "entries"):
+            raise ValueError(f"latent attention: gated {gated!r} unknown (known: True, False, 'entries')")
+        self.gate_entries = gated == "entries"
+        self.scale, self.gated, self.shares_cache, self.window = float(scale), bool(gated), shares_cache, window
+        self.g_size = 0 if not gated else heads * vdim if self.gate_entries else heads
         self.names = dict(zip(("q", "dkv", "norm", "uk", "uv", "g", "o"), names))
         self.q_size = heads * (dim + rot_dim)
         self.q_rank = int(q_rank) if q_rank else 0
@@ -54,7 +59,7 @@ class LatentAttention(Mixer):
         first = self.q_rank or self.q_size           # what the first product makes of the queries
         self.c_off = None if shares_cache else first
         self.g_off = first + (0 if shares_cache else rank + rot_dim)
-        used = self.g_off + (heads if gated else 0)
+        used = self.g_off + self.g_size
         self.proj = Linear(hidden, -(-used // 8) * 8)      # q | down projection | gate in one product (rows padded to 8)
         self.used = used
         self.o = Linear(heads * vdim, hidden)
@@ -93,7 +98,7 @@ class LatentAttention(Mixer):
             for name, spec in self.latent_norm.tensors().items():
                 t[n["norm"] + name] = spec
         if self.gated:
-            t[n["g"]] = TensorSpec((H, self.hidden))
+            t[n["g"]] = TensorSpec((self.g_size, self.hidden))
         return t
 
     def load(self, get):
@@ -154,5 +159,6 @@ class LatentAttention(Mixer):
                                        self.attn_ws, scale=self.scale,
                                        window=self.window or 0, heads=H, rank=R, rot_dim=dr, page_size=self.page_size)
         ops.heads_nt(self.ol_buf, 0, R, self.uv, self.attn_buf, 0, self.vdim, T,
-                     gate=self.proj_buf if self.gated else None, gate_off=self.g_off)
+                     gate=self.proj_buf if self.gated else None, gate_off=self.g_off,
+                     gate_entries=self.gate_entries)
         return self.o.forward(self.attn_buf, self.out_buf, T, scratch=True)

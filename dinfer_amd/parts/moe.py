@@ -21,6 +21,9 @@ weigh as they are. `weigh="input"`: a chosen expert's weight multiplies what goe
 out, y = sum_chosen expert_e(p_e x); the first product is linear in its input, so the weight multiplies its float sums
 before the activation. With one choice a token its expert's row is the layer's output, and nothing is left to sum.
 
+`clamp=(limit, slope)` (gated, without a shared expert): an expert is down_e( g sigmoid(slope g) (u + 1) ) with
+g = min(gate_e x, limit) and u = up_e x clamped to [-limit, limit].
+
 Per step: one kernel routes (logits, choice, weights, the shared gate), one sorts the (token, choice) entries by
 expert and writes the work list of row tiles, two launches run the products of all experts (gate and up with the
 activation, then down, each row computed alone and written to its entry's place), and one sums a token's entries in
@@ -46,7 +49,7 @@ class RoutedExperts(FeedForward):
 
     def __init__(self, hidden: int, experts: int, top: int, intermediate: int, shared_intermediate: int | None = None,
                  act: str = "silu", gated: bool = True, shared_gate: bool = True, scores: str = "chosen",
-                 correction: bool = False, identity: int = 0, weigh: str = "output"):
+                 correction: bool = False, identity: int = 0, weigh: str = "output", clamp: tuple | None = None):
         if gated and act != "silu":
             raise ValueError(f"routed feed-forward: gated activation {act!r} has no kernel (known: ['silu'])")
         if not gated and act not in ops.EXPERT_ACTS:
@@ -54,6 +57,9 @@ class RoutedExperts(FeedForward):
         if weigh not in ("output", "input") or (weigh == "input" and (identity or shared_intermediate)):
             raise ValueError(f"routed feed-forward: weights on the {weigh!r} with {identity} identity experts or a shared one "
                              "are not built (known: 'output', and 'input' for routed experts alone)")
+        if clamp is not None and (not gated or shared_intermediate or not clamp[0] > 0):
+            raise ValueError(f"routed feed-forward: clamp {clamp!r} goes with gated experts, no shared one, and a positive limit")
+        self.clamp = None if clamp is None else (float(clamp[0]), float(clamp[1]))
         self.weigh_input = weigh == "input"
         if scores not in ("chosen", "all", "sigmoid") or identity < 0 or (scores != "all" and (correction or identity)):
             raise ValueError(f"routed feed-forward: scores {scores!r} with correction {correction} and {identity} identity "
@@ -133,7 +139,7 @@ class RoutedExperts(FeedForward):
         ops.moe_scatter(self.idx, n, self.outputs, self.offsets, self.perm, self.tiles, rows, real_experts=self.experts)
         ops.experts_nt(x, self.w_in, self.act_buf, n, self.tiles, self.offsets, self.perm, gated=self.gated, a_div=top,
                        c_to_perm=False, tile_rows=rows, act=None if self.gated else self.act,
-                       row_scale=self.share if self.weigh_input else None)
+                       row_scale=self.share if self.weigh_input else None, clamp=self.clamp)
         alone = self.weigh_input and top == 1      # a token's one row of the second product is its output
         ops.experts_nt(self.act_buf, self.w_out, self.out_buf if alone else self.y_buf, n, self.tiles, self.offsets, self.perm, gated=False, a_div=0,
                        c_to_perm=True, tile_rows=rows)
