@@ -9,6 +9,7 @@
     python bench.py --workload fanulix [--fanulix-shape 2k|4k] [--layers 4] [--prompt 2048] [--only fanulix|karopel|qwen3]
     python bench.py --workload verorax [--verorax-shape 2k|4k] [--layers 4] [--prompt 2048] [--only verorax|kudurax|karopel|qwen3]
     python bench.py --workload lotelix [--lotelix-shape 2k|4k] [--layers 4] [--prompt 2048] [--only lotelix|fanulix|karopel|qwen3]
+    python bench.py --workload dumovik [--dumovik-shape 2k|4k] [--layers 4] [--prompt 2048] [--only dumovik|kudurax|fanulix|qwen3]
 
 Prints ONE JSON line. `value` is decoded tokens per second at the default batch (8), each
 request with a 2,048-token prompt in a 4,096-token context; a "step" is one decode step
@@ -390,6 +391,53 @@ def lotelix(a, torch, Engine, SamplingParams) -> int:
                         LotelixConfig.from_dict(lotelix_config(shape, layers, 32768)), beside=beside)
 
 
+# Dumovik layer sizes that resemble a real model's: a lightning attention of heads of 128 x 128 and a dense gelu feed-forward;
+# latent attention of 512 + 64 a token with a gate an output entry; two attentions with grouped keys and values in chunks of
+# 1,024 positions, the second on the first one's keys; 64 routed experts of which a token uses 6 in every second layer.
+# Beside them Kudurax layers (latent attention, routed experts), Fanulix layers (a linear recurrence with fixed decays) and
+# Qwen3 layers of the same width
+DUMOVIK_SHAPES = {
+    "2k": dict(width=2048, heads=16, kv_heads=4, dim=128, chunk=1024, softcap=50.0, lat_heads=16, rot_dim=64, rank=512, ff=8192,
+               experts=64, top=6, expert_ff=1408, kudurax="2k", fanulix="2k",
+               qwen=dict(num_attention_heads=16, num_key_value_heads=4, head_dim=128, intermediate_size=8192)),
+    "4k": dict(width=4096, heads=32, kv_heads=8, dim=128, chunk=1024, softcap=50.0, lat_heads=32, rot_dim=64, rank=512, ff=12288,
+               experts=64, top=8, expert_ff=1536, kudurax="4k", fanulix="4k",
+               qwen=dict(num_attention_heads=32, num_key_value_heads=8, head_dim=128, intermediate_size=12288)),
+}
+
+
+def dumovik_config(shape: dict, layers: int, vocab: int) -> dict:
+    """Layers in fours: lightning (dense), latent attention (routed), attention (dense), attention on the third's keys (routed)."""
+    d, H = shape["dim"], shape["heads"]
+    dense = dict(kind="dense", ff=shape["ff"])
+    moe = dict(kind="moe", expert=dict(ff=shape["expert_ff"], limit=7.0), router=dict(experts=shape["experts"], top=shape["top"]))
+    lig = dict(heads=H, dim=d, vdim=d, decay=[1.0 - 2.0 ** (-2 - 6 * h / H) for h in range(H)])
+    lat = dict(heads=shape["lat_heads"], dim=d, rot_dim=shape["rot_dim"], vdim=d, kv_rank=shape["rank"],
+               scale=(d + shape["rot_dim"]) ** -0.5, rot=dict(base=1000000.0, dims=shape["rot_dim"]))
+    att = dict(heads=H, kv_heads=shape["kv_heads"], dim=d, vdim=d, scale=d ** -0.5, softcap=shape["softcap"],
+               mask=dict(size=shape["chunk"]))
+    four = [("lightning", lig, dense), ("latent_attention", lat, moe), ("attention", att, dense), ("attention", att, moe)]
+    out = []
+    for i in range(layers):
+        typ, m, mlp = four[i % 4]
+        out.append(dict(type=typ, mixer=dict(m, kv_from=i - 1) if i % 4 == 3 else m, mlp=mlp))
+    return dict(architecture="Dumovik", vocab=vocab, width=shape["width"], norm=dict(eps=1e-5), layers=out)
+
+
+def dumovik(a, torch, Engine, SamplingParams) -> int:
+    """Prefill and decode throughput of Dumovik layers of a real model's sizes beside Kudurax, Fanulix and Qwen3 layers of the
+    same width."""
+    from dinfer_amd.config.dumovik import DumovikConfig
+    from dinfer_amd.config.fanulix import FanulixConfig
+    from dinfer_amd.config.kudurax import KuduraxConfig
+    shape = DUMOVIK_SHAPES[a.dumovik_shape]
+    layers = a.layers or 4
+    beside = {"kudurax": KuduraxConfig.from_dict(kudurax_config(KUDURAX_SHAPES[shape["kudurax"]], layers, 32768)),
+              "fanulix": FanulixConfig.from_dict(fanulix_config(FANULIX_SHAPES[shape["fanulix"]], layers, 32768))}
+    return beside_qwen3(a, torch, Engine, SamplingParams, "dumovik", "Dumovik", a.dumovik_shape, shape,
+                        DumovikConfig.from_dict(dumovik_config(shape, layers, 32768)), beside=beside)
+
+
 def fanulix(a, torch, Engine, SamplingParams) -> int:
     """Prefill and decode throughput of Fanulix layers of a real model's sizes beside Karopel and Qwen3 layers of the same
     width."""
@@ -511,10 +559,11 @@ def main() -> int:
     ap.add_argument("--fanulix-shape", default="2k", choices=sorted(FANULIX_SHAPES), help="fanulix: layer sizes")
     ap.add_argument("--verorax-shape", default="2k", choices=sorted(VERORAX_SHAPES), help="verorax: layer sizes")
     ap.add_argument("--lotelix-shape", default="2k", choices=sorted(LOTELIX_SHAPES), help="lotelix: layer sizes")
-    ap.add_argument("--only", default="", choices=["", "kudurax", "karopel", "fanulix", "verorax", "lotelix", "qwen3"],
-                    help="kudurax, karopel, fanulix, verorax, lotelix: measure one of the models")
+    ap.add_argument("--dumovik-shape", default="2k", choices=sorted(DUMOVIK_SHAPES), help="dumovik: layer sizes")
+    ap.add_argument("--only", default="", choices=["", "kudurax", "karopel", "fanulix", "verorax", "lotelix", "dumovik", "qwen3"],
+                    help="kudurax, karopel, fanulix, verorax, lotelix, dumovik: measure one of the models")
     ap.add_argument("--workload", default="decode", choices=["decode", "serving", "closed", "kudurax", "karopel", "fanulix", "verorax",
-                                                                  "lotelix"],
+                                                                  "lotelix", "dumovik"],
                     help="serving: 32 requests with prompts of 512 to 3,072 tokens fed in portions of 512 beside the "
                          "requests that decode, 256 outputs each (meant for the 14B shape); closed: --concurrency "
                          "requests live at any time, --prompt tokens in and --max-tokens out each, the load of the "
@@ -544,6 +593,8 @@ def main() -> int:
         return verorax(a, torch, Engine, SamplingParams)
     if a.workload == "lotelix":
         return lotelix(a, torch, Engine, SamplingParams)
+    if a.workload == "dumovik":
+        return dumovik(a, torch, Engine, SamplingParams)
     if a.workload == "fanulix":
         return fanulix(a, torch, Engine, SamplingParams)
     if a.workload == "serving":

@@ -39,6 +39,7 @@ SOURCES = {
     "delta": "delta.hip",
     "decay": "decay.hip",
     "linear_attention": "linear_attention.hip",
+    "lightning": "lightning.hip",
     "scan": "scan.hip",
     "streams": "streams.hip",
     "sampling": "sampling.hip",

@@ -60,6 +60,11 @@ SIGNATURES = {
         "linear_attention",
         [_I, _P, _P, _P, _L, _P, _L, _F, _P, _P, _P, _L, _P, _P, _P, _P, _L, _I, _L, _L, _I, _I, _I, _I, _P, _I, _P],
     ),
+    "dinfer_lightning_chunk": ("lightning", []),
+    "dinfer_lightning_supports": ("lightning", [_I, _I, _L]),
+    "dinfer_lightning_cuts": ("lightning", [_L, _L, _I, _I, _I]),
+    "dinfer_lightning": ("lightning", [_P, _P, _P, _L, _P, _P, _P, _L, _P, _P, _P, _P, _L, _I, _L, _L, _I, _I, _I, _I, _P]),
+    "dinfer_lightning_few": ("lightning", [_I, _P, _P, _P, _L, _P, _P, _P, _P, _P, _P, _L, _I, _I, _I, _I, _P]),
     "dinfer_attn_paged_ref": (
         "attention_ref",
         [_I, _P, _L, _P, _L, _P, _P, _P, _L, _P, _P, _I, _L, _F, _I, _I, _I, _I, _I, _P],

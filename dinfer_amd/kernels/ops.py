@@ -620,6 +620,63 @@ def gla_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: tor
     return out
 
 
+# ---- linear attention with constant decays, on the matrix cores ------------------------------------------
+def lightning_supports(dim: int, vdim: int, ld: int) -> bool:
+    return bool(lib.get("dinfer_lightning_supports")(dim, vdim, ld))
+
+
+def lightning_places(tokens: int, reqs: int) -> int:
+    """Chunks whose notes lightning may keep in a step of up to that many tokens and requests."""
+    return tokens // int(lib.get("dinfer_lightning_chunk")()) + reqs + 1
+
+
+def lightning_cuts(tokens: int, max_rows: int, num_reqs: int, heads: int, vdim: int) -> bool:
+    """Whether a step of these counts runs in chunks side by side (a rule of the counts alone)."""
+    return bool(lib.get("dinfer_lightning_cuts")(tokens, max_rows, num_reqs, heads, vdim))
+
+
+def lightning(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, out: torch.Tensor, *,
+              notes: torch.Tensor | None, state_slots: torch.Tensor, cu_seqlens: torch.Tensor, seq_lens: torch.Tensor,
+              num_reqs: int, tokens: int, max_rows: int, cut: bool, heads: int, dim: int, vdim: int) -> torch.Tensor:
+    """Per request and head: S <- decay S + k v^T, out = S^T q, with q, k and v the silu of the operands (bfloat16 column
+    blocks of one buffer, [T, heads dim] and [T, heads vdim]). decay float32 [heads]; state [slots, heads, vdim, dim] float32,
+    updated in place; out [T, heads vdim] float32. cut: in chunks side by side, with scratch notes [places, heads, vdim, dim]
+    (lightning_places of the step at least)."""
+    _need_gpu(q, k, v, decay, state, out, notes, state_slots, cu_seqlens, seq_lens)
+    assert q.dtype == k.dtype == v.dtype == torch.bfloat16 and _rows(q) == _rows(k) == _rows(v)
+    assert decay.dtype == state.dtype == out.dtype == torch.float32 and state.is_contiguous()
+    assert decay.numel() == heads and decay.is_contiguous()
+    assert tuple(state.shape[1:]) == (heads, vdim, dim) and out.shape[1] >= heads * vdim
+    assert q.shape[1] >= heads * dim and k.shape[1] >= heads * dim and v.shape[1] >= heads * vdim
+    assert min(t.shape[0] for t in (q, k, v, out)) >= tokens
+    places = 0
+    if cut:
+        assert notes is not None and notes.dtype == torch.float32 and notes.is_contiguous()
+        places = notes.numel() // (heads * vdim * dim)
+    lib.call("dinfer_lightning", q.data_ptr(), k.data_ptr(), v.data_ptr(), _rows(q), decay.data_ptr(), state.data_ptr(),
+             _ptr(notes) if cut else 0, places, state_slots.data_ptr(), cu_seqlens.data_ptr(), seq_lens.data_ptr(),
+             out.data_ptr(), _rows(out), num_reqs, tokens, max_rows, int(cut), heads, dim, vdim, _stream())
+    return out
+
+
+def lightning_few(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, out: torch.Tensor, *,
+                  state_slots: torch.Tensor, cu_seqlens: torch.Tensor, seq_lens: torch.Tensor, num_reqs: int, tokens: int,
+                  heads: int, dim: int, vdim: int) -> torch.Tensor:
+    """The rule of lightning() token by token, for steps whose portions bring a few rows each: any storage type, dim a
+    multiple of 4."""
+    _need_gpu(q, k, v, decay, state, out, state_slots, cu_seqlens, seq_lens)
+    assert q.dtype == k.dtype == v.dtype and _rows(q) == _rows(k) == _rows(v)
+    assert decay.dtype == state.dtype == out.dtype == torch.float32 and state.is_contiguous()
+    assert decay.numel() == heads and decay.is_contiguous()
+    assert tuple(state.shape[1:]) == (heads, vdim, dim) and out.shape[1] >= heads * vdim
+    assert q.shape[1] >= heads * dim and k.shape[1] >= heads * dim and v.shape[1] >= heads * vdim
+    assert min(t.shape[0] for t in (q, k, v, out)) >= tokens
+    lib.call("dinfer_lightning_few", dtype_code(q.dtype), q.data_ptr(), k.data_ptr(), v.data_ptr(), _rows(q), decay.data_ptr(),
+             state.data_ptr(), state_slots.data_ptr(), cu_seqlens.data_ptr(), seq_lens.data_ptr(), out.data_ptr(), _rows(out),
+             num_reqs, heads, dim, vdim, _stream())
+    return out
+
+
 # ---- gated recurrence of single channels ---------------------------------------------------------------
 def min_gru_places(tokens: int, reqs: int) -> int:
     """Chunks whose notes min_gru may keep in a step of up to that many tokens and requests."""

@@ -109,7 +109,7 @@ class Attention(Mixer):
                                   or POSITION_ENCODINGS.get(position.kind) is not POSITION_ENCODINGS.get("none")):
             raise ValueError("attention: a layer that reads another one's keys takes norms over the whole projection or none, and "
                              "no biases, rotation, or values of another kind")
-        if self.chunk and self.keep_first and not window:
+        if self.chunk and keep_first:
             raise ValueError("attention: kept first keys beside chunks are not built")
         # the keys the cache keeps: those of the window, or of a chunk as long as it may reach back
         own = min((n for n in (window, self.chunk) if n), default=None)

@@ -8,8 +8,9 @@ With x the mixer's input, H heads:
     y = Wo ( o / rms(o) * w * sigmoid(Wg x) )                        (the root mean square over all heads' entries at once)
 
 One product makes q | k | v | gate. The state lives in the request's state slot (DeltaStateSpec without a convolution); a
-request's first step (position 0) starts from zeros. Steps with prompt portions run in chunks of tokens on the matrix
-cores where the sizes fit (ops.lightning_chunks), everything else token by token (ops.gla_recurrence with fixed decays).
+request's first step (position 0) starts from zeros. bfloat16 steps with prompt portions run in blocks of tokens on the
+matrix cores (ops.lightning), steps whose portions bring a few rows token by token (ops.lightning_few), 32-bit prompts and
+sizes those two do not take through ops.gla_recurrence with fixed decays.
 """
 from __future__ import annotations
 
@@ -20,6 +21,8 @@ from .base import CacheView, Mixer
 from .linear import Linear
 from .registry import MIXERS
 from .spec import DeltaStateSpec, TensorSpec
+
+FEW_ROWS = 8      # the longest portion of a step up to which its tokens are taken one by one
 
 
 @MIXERS.register("lightning")
@@ -67,11 +70,13 @@ class Lightning(Mixer):
         self.o_buf = ws.buffer("lightning_o", self.v_size, dtype=torch.float32)
         self.gated_buf = ws.buffer("lightning_gated", self.v_size)
         self.out_buf = ws.buffer("mixer_out", self.hidden)
-        places = ops.gla_places(ctx.max_tokens, ctx.max_reqs)
+        self.blocks = ctx.dtype == torch.bfloat16 and ops.lightning_supports(self.dim, self.vdim, self.proj.out_features)
+        places = (ops.lightning_places if self.blocks else ops.gla_places)(ctx.max_tokens, ctx.max_reqs)
         self.notes = self.products = None
         if places > ctx.max_reqs + 1:      # (an engine whose longest step is shorter than a chunk cuts none)
             self.notes = ws.buffer("lightning_notes", self.heads * self.vdim * self.dim, dtype=torch.float32, rows=places)
-            self.products = ws.buffer("lightning_products", self.qk_size, dtype=torch.float32, rows=places)
+            if not self.blocks:
+                self.products = ws.buffer("lightning_products", self.qk_size, dtype=torch.float32, rows=places)
 
     def forward(self, x, batch, cache: CacheView):
         T, qk, H = batch.num_tokens, self.qk_size, self.heads
@@ -79,11 +84,19 @@ class Lightning(Mixer):
         if not cache.owner:
             raise NotImplementedError("a recurrent mixer keeps a state a request: an entry that borrows a cache has none")
         self.proj.forward(x, p, T, scratch=True)
-        cut = self.notes is not None and ops.gla_cuts(T, batch.max_q_len, batch.num_reqs, H, self.vdim)
-        ops.gla_recurrence(p[:, :qk], p[:, qk:2 * qk], p[:, 2 * qk:self.g_off], None, cache.state, self.o_buf, q_scale=1.0,
-                           notes=self.notes, products=self.products, state_slots=batch.state_slots, cu_seqlens=batch.cu_seqlens,
-                           seq_lens=batch.seq_lens, num_reqs=batch.num_reqs, tokens=T, max_rows=batch.max_q_len, cut=cut, heads=H,
-                           dim=self.dim, vdim=self.vdim, fixed=self.decay_vec, act=True)
+        q, k, v = p[:, :qk], p[:, qk:2 * qk], p[:, 2 * qk:self.g_off]
+        step = dict(state_slots=batch.state_slots, cu_seqlens=batch.cu_seqlens, seq_lens=batch.seq_lens, num_reqs=batch.num_reqs,
+                    tokens=T, heads=H, dim=self.dim, vdim=self.vdim)
+        if self.dim % 4 == 0 and batch.max_q_len <= FEW_ROWS:
+            ops.lightning_few(q, k, v, self.decay_vec, cache.state, self.o_buf, **step)
+        elif self.blocks:
+            cut = self.notes is not None and ops.lightning_cuts(T, batch.max_q_len, batch.num_reqs, H, self.vdim)
+            ops.lightning(q, k, v, self.decay_vec, cache.state, self.o_buf, notes=self.notes, cut=cut, max_rows=batch.max_q_len,
+                          **step)
+        else:
+            cut = self.products is not None and ops.gla_cuts(T, batch.max_q_len, batch.num_reqs, H, self.vdim)
+            ops.gla_recurrence(q, k, v, None, cache.state, self.o_buf, q_scale=1.0, notes=self.notes, products=self.products,
+                               fixed=self.decay_vec, act=True, cut=cut, max_rows=batch.max_q_len, **step)
         ops.gated_group_norm(self.o_buf, p, self.g_off, self.gated_buf, T, groups=1, group=self.v_size, eps=self.norm_eps,
                              weight=self.gain, gate_first=False, gate="sigmoid")
         return self.o.forward(self.gated_buf, self.out_buf, T, scratch=True)
